@@ -68,6 +68,8 @@ _PROTOS = {
     "nv_stage_decode_inputs": (_i, [_p, _p, _p, _p, _p, _i, _p, _p, _p, _p, _p, _i, _i, _i, _p]),
     "nv_linear": (_i, [_p, _i64, _p, _p, _i64, _p, _p, _i64, _i, _i64, _i, _i, _i, _i64, _i64, _i64, _i64, _p, _i, _i, _p,
                        _i64, _f, _i, _p]),
+    "nv_linear_scaled": (_i, [_p, _i64, _p, _p, _i64, _p, _p, _i64, _i, _i64, _i, _i, _i, _i64, _i64, _i64, _i64, _p, _i, _i,
+                              _p, _i64, _f, _p, _i, _p]),
     "nv_embed_scale": (_i, [_p, _p, _p, _i64, _i, _i64, _f, _i, _p]),
     "nv_dyt_norm": (_i, [_p, _p, _i64, _p, _p, _p, _p, _p, _i64, _i, _i, _p]),
     "nv_gated_postnorm_add": (_i, [_p, _p, _i64, _p, _p, _i64, _p, _p, _p, _i64, _i64, _i, _f, _f, _i, _p]),
@@ -75,8 +77,10 @@ _PROTOS = {
     "nv_gated_postnorm_add_conv": (_i, [_p, _p, _i64, _p, _p, _i64, _p, _p, _p, _i64, _i64, _i, _f, _f, _p, _i, _p, _p, _p,
                                         _p, _i64, _i, _p]),
     "nv_bias_act_f32": (_i, [_p, _p, _i, _p, _i64, _i, _p, _f, _i, _p]),
+    "nv_sandwich_norm": (_i, [_p, _p, _i64, _p, _p, _p, _p, _i64, _p, _p, _i, _p, _p, _i64, _p, _p, _i64, _i64, _i, _f, _i, _p]),
     "nv_rmsnorm_f32": (_i, [_p, _i64, _p, _p, _i64, _i64, _i, _f, _i, _p]),
     "nv_act_mul_f32": (_i, [_p, _p, _i64, _i, _i, _f, _i, _p]),
+    "nv_bias_act_mul_f32": (_i, [_p, _p, _p, _i64, _i, _i, _f, _i, _p]),
     "nv_act_f32": (_i, [_p, _p, _i64, _i, _p, _f, _i, _p]),
     "nv_sample_f32": (_i, [_p, _i64, _p, _p, _i, _i, _u64, _p]),
     "nv_gla_recurrent": (_i, [_p, _i64, _i, _i, _i, _i, _p, _i64, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _f, _f, _f, _i, _p]),
@@ -94,6 +98,7 @@ _PROTOS = {
     "nv_latent_expand": (_i, [_p, _p, _p, _i64, _i, _i, _i, _i, _i, _i, _p]),
     "nv_moe_route": (_i, [_p, _i64, _p, _p, _i64, _i, _i, _i, _p]),
     "nv_moe_sort": (_i, [_p, _i64, _i, _i, _p, _p, _p, _p]),
+    "nv_moe_plan": (_i, [_p, _i64, _i64, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p]),
     "nv_moe_combine": (_i, [_p, _p, _p, _i, _p, _p, _i64, _p, _i64, _i, _p]),
     "nv_embed_sinusoid": (_i, [_p, _p, _p, _p, _p, _i64, _i, _i, _i64, _i, _p]),
     "nv_hc_norm": (_i, [_p, _i, _i, _p, _i64, _p, _p, _p, _i, _f, _p, _p, _i64, _i, _i64, _i, _p]),
@@ -102,9 +107,9 @@ _PROTOS = {
     "nv_qk_norm_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _p, _f, _f, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
     "nv_window_attn": (_i, [_p, _p, _p, _i, _p, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
     "nv_qk_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _p, _p, _f, _i, _f, _f, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
-    "nv_paged_softmax_attn": (_i, [_p, _p, _p, _i, _p, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i,
+    "nv_paged_softmax_attn": (_i, [_p, _p, _p, _i, _p, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i,
                                    _i, _p, _p, _i64, _i, _p, _sz, _i, _p]),
-    "nv_qk_rotate_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _i, _p, _p, _f, _i, _p, _i, _f, _p, _i64, _p, _f, _f, _p,
+    "nv_qk_rotate_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _i, _p, _p, _f, _i, _p, _i, _i, _f, _p, _i64, _p, _f, _f, _p,
                                 _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
     "nv_paged_softmax_attn_workspace_bytes": (_sz, [_i64, _i, _i, _i, _i]),
     "nv_causal_conv": (_i, [_p, _p, _i64, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i, _i, _i, _p]),

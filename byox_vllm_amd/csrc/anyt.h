@@ -22,6 +22,7 @@ __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)
 __device__ __forceinline__ float gelu_tanh_f32(float z) {
   return 0.5f * z * (1.0f + tanhf(0.7978845608028654f * (z + 0.044715f * z * z * z)));
 }
+__device__ __forceinline__ float gelu_erf_f32(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)); }
 // Gated unit act(gate) * up.  act 0: SiLU, 1: tanh-form GELU, 2: the clamped form with limit c,
 // g = min(gate, c), u = clamp(up, -c, c), g * sigmoid(1.702 g) * (u + 1).
 __device__ __forceinline__ float glu_act(float g, float u, int act, float c) {

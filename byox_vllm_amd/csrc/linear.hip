@@ -32,17 +32,20 @@ struct LinArgs {
   float epi_c;
   int act;
   int vec_a, vec_w;
+  const float* row_scale;    // [output rows] factor of the product, ahead of bias and epilogue, or null
 };
 
 enum { EPI_NONE = 0, EPI_GLU = 1, EPI_SOFTCAP = 2, EPI_ROW_GATE = 3, EPI_ACT = 4 };
 
 // EPI_ACT: an element-wise function of the product.  act 0 SiLU, 1 tanh-form GELU, 2 xIELU with its two positive
-// coefficients at epi_ptr (a z^2 + z/2 above zero, b (exp(z) - 1 - z) + z/2 below), 3 multiplication by epi_c.
+// coefficients at epi_ptr (a z^2 + z/2 above zero, b (exp(z) - 1 - z) + z/2 below), 3 multiplication by epi_c, 4 erf-form
+// GELU.
 __device__ __forceinline__ float unary_act(float v, int act, const float* prm, float c) {
   switch (act) {
     case 0: return silu_f32(v);
     case 1: return gelu_tanh_f32(v);
     case 2: return v > 0.0f ? prm[0] * v * v + 0.5f * v : prm[1] * (expm1f(v) - v) + 0.5f * v;
+    case 4: return gelu_erf_f32(v);
     default: return v * c;
   }
 }
@@ -158,14 +161,16 @@ __global__ __launch_bounds__(256) void linear_kernel(LinArgs p) {
   for (int i = 0; i < 4; ++i) {
     const int64_t s = mbase + 16 * i + c;
     if (i >= nsub || s >= hi) continue;
+    const float rsc = p.row_scale ? p.row_scale[s] : 1.0f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int n = n0 + 4 * g + r;
       if (n >= p.N) continue;
-      float v = acc[i][r];
+      float v = acc[i][r] * rsc;
       if (bias) v += ld_f32<T>(bias + n);
       if constexpr (EPI == EPI_GLU) {
-        const float u = accu[i][r];
+        float u = accu[i][r] * rsc;
+        if (bias) u += ld_f32<T>(bias + p.N + n);
         v = glu_act(v, u, p.act, p.epi_c);
       } else if constexpr (EPI == EPI_SOFTCAP) {
         v = p.epi_c * tanhf(v / p.epi_c);
@@ -292,16 +297,19 @@ __global__ __launch_bounds__(256) void linear_tile_kernel(LinArgs p) {
   for (int i = 0; i < 4; ++i) {
     const int64_t s = mbase + 64 * wm + 16 * i + c;
     if (s >= hi) continue;
+    const float rsc = p.row_scale ? p.row_scale[s] : 1.0f;
 #pragma unroll
     for (int j = 0; j < NJ; ++j) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int n = n0 + (GLU ? 32 * wn : 64 * wn) + 16 * j + 4 * g + r;
         if (n >= p.N) continue;
-        float v = acc[i][j][r];
+        float v = acc[i][j][r] * rsc;
         if (bias) v += ld_f32<bf16_t>(bias + n);
         if constexpr (GLU) {
-          v = glu_act(v, accu[i][j][r], p.act, p.epi_c);
+          float u = accu[i][j][r] * rsc;
+          if (bias) u += ld_f32<bf16_t>(bias + p.N + n);
+          v = glu_act(v, u, p.act, p.epi_c);
         } else if constexpr (EPI == EPI_SOFTCAP) {
           v = p.epi_c * tanhf(v / p.epi_c);
         } else if constexpr (EPI == EPI_ROW_GATE) {
@@ -404,15 +412,17 @@ __global__ __launch_bounds__(256) void linear_fewrow_kernel(LinArgs p) {
   for (int i = 0; i < NSUB; ++i) {
     const int64_t s = lo + 16 * i + c;
     if (i >= nsub || s >= hi) continue;
+    const float rsc = p.row_scale ? p.row_scale[s] : 1.0f;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int n = n0 + 4 * g + r;
       if (n >= p.N) continue;
       const int e = 4 * lane + r;
-      float v = part[0][0][i][e] + part[0][1][i][e] + part[0][2][i][e] + part[0][3][i][e];
+      float v = (part[0][0][i][e] + part[0][1][i][e] + part[0][2][i][e] + part[0][3][i][e]) * rsc;
       if (bias) v += ld_f32<T>(bias + n);
       if constexpr (GLU) {
-        const float u = part[1][0][i][e] + part[1][1][i][e] + part[1][2][i][e] + part[1][3][i][e];
+        float u = (part[1][0][i][e] + part[1][1][i][e] + part[1][2][i][e] + part[1][3][i][e]) * rsc;
+        if (bias) u += ld_f32<T>(bias + p.N + n);
         v = glu_act(v, u, p.act, p.epi_c);
       } else if constexpr (EPI == EPI_SOFTCAP) {
         v = p.epi_c * tanhf(v / p.epi_c);
@@ -468,13 +478,24 @@ extern "C" int nv_linear(const void* a, int64_t a_row_stride, const int32_t* a_r
                          int batch, int64_t a_batch_stride, int64_t w_batch_stride, int64_t out_batch_stride,
                          int64_t bias_batch_stride, const int32_t* group_offsets, int epilogue, int act,
                          const float* epi_ptr, int64_t epi_row_stride, float epi_const, int dtype, nv_stream_t stream) {
+  return nv_linear_scaled(a, a_row_stride, a_rows, w, w_row_stride, bias, out, out_row_stride, out_dtype, M, N, K, batch,
+                          a_batch_stride, w_batch_stride, out_batch_stride, bias_batch_stride, group_offsets, epilogue, act,
+                          epi_ptr, epi_row_stride, epi_const, nullptr, dtype, stream);
+}
+
+extern "C" int nv_linear_scaled(const void* a, int64_t a_row_stride, const int32_t* a_rows, const void* w, int64_t w_row_stride,
+                         const void* bias, void* out, int64_t out_row_stride, int out_dtype, int64_t M, int N, int K,
+                         int batch, int64_t a_batch_stride, int64_t w_batch_stride, int64_t out_batch_stride,
+                         int64_t bias_batch_stride, const int32_t* group_offsets, int epilogue, int act,
+                         const float* epi_ptr, int64_t epi_row_stride, float epi_const, const float* row_scale, int dtype,
+                         nv_stream_t stream) {
   NV_CHECK_ARG(a && w && out, "nv_linear: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_linear: dtype %d is neither bf16 nor fp32", dtype);
   NV_CHECK_ARG(out_dtype == NV_BF16 || out_dtype == NV_F32, "nv_linear: bad output dtype %d", out_dtype);
   NV_CHECK_ARG(M >= 0 && N > 0 && K > 0 && batch > 0 && batch <= 65535, "nv_linear: bad shape M=%lld N=%d K=%d batch=%d",
                (long long)M, N, K, batch);
   NV_CHECK_ARG(epilogue >= EPI_NONE && epilogue <= EPI_ACT, "nv_linear: bad epilogue %d", epilogue);
-  NV_CHECK_ARG(epilogue != EPI_ACT || (act >= 0 && act <= 3 && (act != 2 || epi_ptr)), "nv_linear: bad activation %d", act);
+  NV_CHECK_ARG(epilogue != EPI_ACT || (act >= 0 && act <= 4 && (act != 2 || epi_ptr)), "nv_linear: bad activation %d", act);
   NV_CHECK_ARG(epilogue != EPI_ROW_GATE || epi_ptr, "nv_linear: the row-gate epilogue needs its gate rows");
   NV_CHECK_ARG(epilogue != EPI_SOFTCAP || epi_const > 0.0f, "nv_linear: the soft cap must be positive");
   if (M == 0) return NV_OK;
@@ -484,7 +505,7 @@ extern "C" int nv_linear(const void* a, int64_t a_row_stride, const int32_t* a_r
   const int per = dtype == NV_BF16 ? 8 : 4;
   LinArgs p{a, a_row_stride, a_rows, w, w_row_stride, bias, out, out_row_stride, M, N, K, a_batch_stride,
             w_batch_stride, out_batch_stride, bias_batch_stride, group_offsets, epi_ptr, epi_row_stride, epi_const, act,
-            0, 0};
+            0, 0, row_scale};
   p.vec_a = (uintptr_t)a % 16 == 0 && a_row_stride % per == 0 && (a_batch_stride * esz) % 16 == 0;
   p.vec_w = (uintptr_t)w % 16 == 0 && w_row_stride % per == 0 && (w_batch_stride * esz) % 16 == 0;
   dim3 grid((unsigned)((N + 63) / 64), (unsigned)mtiles, (unsigned)batch);

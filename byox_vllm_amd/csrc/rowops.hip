@@ -195,6 +195,161 @@ __global__ __launch_bounds__(256) void gated_postnorm_add_kernel(float* __restri
   }
 }
 
+// A sublayer normed on both sides: the previous sublayer's result joins the residual through its output norm, and the
+// next sublayer's input norm reads the new row.  The result may be a plain row (plus the bias its last product left
+// out) or the rows of a mixture's experts, gathered, weighted and summed here.
+struct SandwichArgs {
+  float* x;                  // [.., n] residual
+  const float* y;            // [.., y_rs] plain rows, or expert rows [.., n] addressed by slot_of; null: nothing joins
+  int64_t y_rs;
+  const void* y_bias;        // [n] or null
+  const void* w_post;        // [n]; null: the result is added as it is
+  const void* w_pre;         // [n]; null: no output
+  void* out;
+  int64_t out_rs;
+  const int32_t* rows_idx;   // output row i comes from row rows_idx[i], x is left alone; null: row i, x is updated
+  const int32_t* slot_of;    // [.., choices] or null
+  int choices;
+  const float* weights;      // [.., choices] or null (all 1)
+  const float* last_gate;    // logits [.., last_gate_rs]: the last choice is weighed by their sigmoid; or null
+  int64_t last_gate_rs;
+  const float* shared;       // [.., n] more rows to add, times sigmoid(shared_gate), or null
+  const float* shared_gate;
+  int64_t shared_gate_rs;
+  int n;
+  float eps;
+};
+
+// NV > 0: rows of at most NV * 1024 numbers, a multiple of 4, everything 16-byte aligned: a thread keeps its numbers in
+// registers from the load to the last norm.  NV == 0: any row; the numbers wait in LDS.
+template <typename T, int NV>
+__global__ __launch_bounds__(256) void sandwich_norm_kernel(SandwichArgs p) {
+  extern __shared__ float row_lds[];
+  __shared__ float red[32];
+  constexpr int V = NV > 0 ? 4 : 1, STEPS = NV > 0 ? NV : 1;
+  typedef typename Pack4<T>::type P;
+  const int64_t i = blockIdx.x, t = p.rows_idx ? p.rows_idx[i] : i;
+  const int n = p.n, tid = threadIdx.x;
+  float* xr = p.x + t * n;
+  const float gate = p.shared ? sigmoid_f32(p.shared_gate[t * p.shared_gate_rs]) : 0.0f;
+  const float last = p.slot_of && p.last_gate ? sigmoid_f32(p.last_gate[t * p.last_gate_rs]) : 1.0f;
+  f32x4 v[STEPS];
+  auto load4 = [](const float* q, int c) { return *reinterpret_cast<const f32x4*>(q + c); };
+  auto widen4 = [](const void* q, int c) { return Pack4<T>::widen(*reinterpret_cast<const P*>(reinterpret_cast<const T*>(q) + c)); };
+  auto factor = [&](int k) {
+    float f = p.weights ? p.weights[t * p.choices + k] : 1.0f;
+    return k == p.choices - 1 && p.last_gate ? last : f;
+  };
+  float ss = 0.0f;
+  if (p.y) {
+    if constexpr (NV > 0) {
+#pragma unroll
+      for (int k = 0; k < STEPS; ++k) v[k] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+      if (p.slot_of) {
+        for (int q = 0; q < p.choices; ++q) {
+          const float f = factor(q);
+          const float* yr = p.y + (int64_t)p.slot_of[t * p.choices + q] * p.y_rs;
+#pragma unroll
+          for (int k = 0; k < STEPS; ++k) {
+            const int c = (tid + k * 256) * 4;
+            if (c < n) {
+              const f32x4 a = load4(yr, c);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) v[k][e] += f * a[e];
+            }
+          }
+        }
+      } else {
+#pragma unroll
+        for (int k = 0; k < STEPS; ++k) {
+          const int c = (tid + k * 256) * 4;
+          if (c < n) v[k] = load4(p.y + t * p.y_rs, c);
+        }
+      }
+#pragma unroll
+      for (int k = 0; k < STEPS; ++k) {
+        const int c = (tid + k * 256) * 4;
+        if (c >= n) continue;
+        if (p.shared) {
+          const f32x4 a = load4(p.shared + t * n, c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[k][e] += gate * a[e];
+        }
+        if (p.y_bias) {
+          const f32x4 b = widen4(p.y_bias, c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[k][e] += b[e];
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += v[k][e] * v[k][e];
+      }
+    } else {
+      for (int c = tid; c < n; c += 256) {
+        float a = 0.0f;
+        if (p.slot_of) {
+          for (int q = 0; q < p.choices; ++q) a += factor(q) * p.y[(int64_t)p.slot_of[t * p.choices + q] * p.y_rs + c];
+        } else {
+          a = p.y[t * p.y_rs + c];
+        }
+        if (p.shared) a += gate * p.shared[t * n + c];
+        if (p.y_bias) a += ld_f32<T>(reinterpret_cast<const T*>(p.y_bias) + c);
+        row_lds[c] = a;
+        ss += a * a;
+      }
+    }
+  }
+  float inv = 1.0f;
+  if (p.y && p.w_post) inv = 1.0f / sqrtf(block_sum(ss, red) / (float)n + p.eps);
+  ss = 0.0f;
+#pragma unroll
+  for (int k = 0; k < STEPS; ++k) {
+    for (int c = (tid + k * 256) * V; c < n; c += NV > 0 ? n : 256) {       // NV > 0: one round
+      if constexpr (NV > 0) {
+        f32x4 a = load4(xr, c);
+        if (p.y) {
+          if (p.w_post) {
+            const f32x4 w = widen4(p.w_post, c);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) a[e] += v[k][e] * inv * w[e];
+          } else {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) a[e] += v[k][e];
+          }
+          if (!p.rows_idx) *reinterpret_cast<f32x4*>(xr + c) = a;
+        }
+        v[k] = a;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += a[e] * a[e];
+      } else {
+        float a = xr[c];
+        if (p.y) {
+          a += row_lds[c] * (p.w_post ? inv * ld_f32<T>(reinterpret_cast<const T*>(p.w_post) + c) : 1.0f);
+          if (!p.rows_idx) xr[c] = a;
+        }
+        row_lds[c] = a;
+        ss += a * a;
+      }
+    }
+  }
+  if (!p.w_pre) return;
+  inv = 1.0f / sqrtf(block_sum(ss, red) / (float)n + p.eps);
+  T* out = reinterpret_cast<T*>(p.out) + i * p.out_rs;
+#pragma unroll
+  for (int k = 0; k < STEPS; ++k) {
+    for (int c = (tid + k * 256) * V; c < n; c += NV > 0 ? n : 256) {
+      if constexpr (NV > 0) {
+        const f32x4 w = widen4(p.w_pre, c);
+        f32x4 a = v[k];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) a[e] = a[e] * inv * w[e];
+        *reinterpret_cast<P*>(out + c) = Pack4<T>::narrow(a);
+      } else {
+        st_f32<T>(out + c, row_lds[c] * inv * ld_f32<T>(reinterpret_cast<const T*>(p.w_pre) + c));
+      }
+    }
+  }
+}
+
 // out[t] = [x[t] | x0[t]] in the storage type; x takes delta first
 template <typename T>
 __global__ __launch_bounds__(256) void residual_pair_kernel(float* __restrict__ x, const float* __restrict__ delta,
@@ -212,15 +367,34 @@ __global__ __launch_bounds__(256) void residual_pair_kernel(float* __restrict__ 
   }
 }
 
-// out[m][j] = act(y[m][j]) * y[m][n + j]: the gated unit's activation over a plain product's [gate | up] rows
-template <typename T>
-__global__ __launch_bounds__(256) void act_mul_f32_kernel(const float* __restrict__ y, T* __restrict__ out, int64_t total,
-                                                          int n, int act, float c) {
-  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
-    const int64_t m = i / n;
+// out[m][j] = act(y[m][j] + b[j]) * (y[m][n + j] + b[n + j]): the gated unit over a plain product's [gate | up] rows
+// (b null: no bias); V numbers per thread and access
+template <typename T, int V>
+__global__ __launch_bounds__(256) void act_mul_f32_kernel(const float* __restrict__ y, const T* __restrict__ bias,
+                                                          T* __restrict__ out, int64_t total, int n, int act, float c) {
+  for (int64_t q = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; q < total / V; q += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t i = q * V, m = i / n;
     const int j = (int)(i - m * n);
-    const float g = y[m * 2 * n + j], u = y[m * 2 * n + n + j];
-    st_f32<T>(out + i, glu_act(g, u, act, c));
+    if constexpr (V == 4) {
+      typedef typename Pack4<T>::type P;
+      f32x4 g = *reinterpret_cast<const f32x4*>(y + m * 2 * n + j), u = *reinterpret_cast<const f32x4*>(y + m * 2 * n + n + j);
+      if (bias) {
+        const f32x4 bg = Pack4<T>::widen(*reinterpret_cast<const P*>(bias + j));
+        const f32x4 bu = Pack4<T>::widen(*reinterpret_cast<const P*>(bias + n + j));
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          g[e] += bg[e];
+          u[e] += bu[e];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) g[e] = glu_act(g[e], u[e], act, c);
+      *reinterpret_cast<P*>(out + i) = Pack4<T>::narrow(g);
+    } else {
+      const float g = y[m * 2 * n + j] + (bias ? ld_f32<T>(bias + j) : 0.0f);
+      const float u = y[m * 2 * n + n + j] + (bias ? ld_f32<T>(bias + n + j) : 0.0f);
+      st_f32<T>(out + i, glu_act(g, u, act, c));
+    }
   }
 }
 
@@ -237,6 +411,7 @@ __global__ __launch_bounds__(256) void act_f32_kernel(const float* __restrict__ 
       case 0: r = silu_f32(v); break;
       case 1: r = gelu_tanh_f32(v); break;
       case 2: r = v > 0.0f ? a * v * v + 0.5f * v : b * (expm1f(v) - v) + 0.5f * v; break;
+      case 4: r = gelu_erf_f32(v); break;
       default: r = v * c; break;
     }
     st_f32<T>(out + i, r);
@@ -306,6 +481,35 @@ extern "C" int nv_sample_f32(const float* logits, int64_t row_stride, const floa
   return NV_OK;
 }
 
+extern "C" int nv_sandwich_norm(float* x, const float* y, int64_t y_row_stride, const void* y_bias, const void* w_post,
+                                const void* w_pre, void* out, int64_t out_row_stride, const int32_t* rows_idx,
+                                const int32_t* slot_of, int choices, const float* weights, const float* last_gate,
+                                int64_t last_gate_stride, const float* shared, const float* shared_gate,
+                                int64_t shared_gate_stride, int64_t rows, int n, float eps, int dtype, nv_stream_t stream) {
+  NV_CHECK_ARG(x && (y || !(y_bias || w_post || slot_of || shared)), "nv_sandwich_norm: null pointer");
+  NV_CHECK_ARG((w_pre == nullptr) == (out == nullptr) && (w_pre || (y && !rows_idx)), "nv_sandwich_norm: nothing to do");
+  NV_CHECK_ARG(!slot_of || choices > 0, "nv_sandwich_norm: bad choices %d", choices);
+  NV_CHECK_ARG(!shared || shared_gate, "nv_sandwich_norm: shared rows need their gate");
+  NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_sandwich_norm: bad dtype %d", dtype);
+  NV_CHECK_ARG(rows >= 0 && rows < (1ll << 31) && n > 0 && n <= 16000, "nv_sandwich_norm: bad shape, rows of %d numbers", n);
+  if (rows == 0) return NV_OK;
+  SandwichArgs p{x, y, y_row_stride, y_bias, w_post, w_pre, out, out_row_stride, rows_idx, slot_of, choices, weights,
+                 last_gate, last_gate_stride, shared, shared_gate, shared_gate_stride, n, eps};
+  auto al16 = [](const void* q) { return ((uintptr_t)q & 15) == 0; };
+  const bool vec = n % 4 == 0 && n <= 4096 && al16(x) && al16(y) && al16(y_bias) && al16(w_post) && al16(w_pre) && al16(out) &&
+                   al16(shared) && (!y || y_row_stride % 4 == 0) && out_row_stride % 4 == 0;
+  hipStream_t s = (hipStream_t)stream;
+#define NV_SANDWICH(NVAL, LDS) \
+  NV_DISPATCH_T(dtype, sandwich_norm_kernel<T, NVAL><<<dim3((unsigned)rows), dim3(256), LDS, s>>>(p))
+  if (vec && n <= 1024) NV_SANDWICH(1, 0);
+  else if (vec && n <= 2048) NV_SANDWICH(2, 0);
+  else if (vec) NV_SANDWICH(4, 0);
+  else NV_SANDWICH(0, (size_t)n * sizeof(float));
+#undef NV_SANDWICH
+  NV_CHECK_LAUNCH();
+  return NV_OK;
+}
+
 extern "C" int nv_residual_pair(float* x, const float* delta, int64_t delta_row_stride, const float* x0, void* out,
                                 int64_t rows, int n, int dtype, nv_stream_t stream) {
   NV_CHECK_ARG(x && x0 && out, "nv_residual_pair: null pointer");
@@ -320,15 +524,25 @@ extern "C" int nv_residual_pair(float* x, const float* delta, int64_t delta_row_
 
 extern "C" int nv_act_mul_f32(const float* y, void* out, int64_t rows, int n, int act, float c, int dtype,
                               nv_stream_t stream) {
+  return nv_bias_act_mul_f32(y, nullptr, out, rows, n, act, c, dtype, stream);
+}
+
+extern "C" int nv_bias_act_mul_f32(const float* y, const void* bias, void* out, int64_t rows, int n, int act, float c,
+                                   int dtype, nv_stream_t stream) {
   NV_CHECK_ARG(y && out, "nv_act_mul_f32: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_act_mul_f32: bad dtype %d", dtype);
   NV_CHECK_ARG(rows >= 0 && n > 0 && act >= 0 && act <= 2 && (act != 2 || c > 0.0f), "nv_act_mul_f32: bad shape or activation");
   if (rows == 0) return NV_OK;
   const int64_t total = rows * n;
-  int64_t blocks = (total + 255) / 256;
+  const bool vec = n % 4 == 0 && ((uintptr_t)y & 15) == 0 && ((uintptr_t)bias & 15) == 0 && ((uintptr_t)out & 15) == 0;
+  int64_t blocks = (total / (vec ? 4 : 1) + 255) / 256;
   if (blocks > 8192) blocks = 8192;
-  NV_DISPATCH_T(dtype, act_mul_f32_kernel<T><<<dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream>>>(
-                           y, (T*)out, total, n, act, c));
+  if (vec)
+    NV_DISPATCH_T(dtype, act_mul_f32_kernel<T, 4><<<dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream>>>(
+                             y, (const T*)bias, (T*)out, total, n, act, c));
+  else
+    NV_DISPATCH_T(dtype, act_mul_f32_kernel<T, 1><<<dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream>>>(
+                             y, (const T*)bias, (T*)out, total, n, act, c));
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
@@ -342,7 +556,7 @@ extern "C" int nv_bias_act_f32(const float* y, const void* bias, int n, void* ou
                                const float* params, float c, int dtype, nv_stream_t stream) {
   NV_CHECK_ARG(y && out && n > 0, "nv_act_f32: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_act_f32: bad dtype %d", dtype);
-  NV_CHECK_ARG(total >= 0 && act >= 0 && act <= 3 && (act != 2 || params), "nv_act_f32: bad shape or activation");
+  NV_CHECK_ARG(total >= 0 && act >= 0 && act <= 4 && (act != 2 || params), "nv_act_f32: bad shape or activation");
   if (total == 0) return NV_OK;
   int64_t blocks = (total + 255) / 256;
   if (blocks > 16384) blocks = 16384;

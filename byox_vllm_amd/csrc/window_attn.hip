@@ -4,7 +4,8 @@
 // over the keys 0 <= i - j < window (window 0: every earlier key).  q arrives already normalised and multiplied by its
 // scale and per-head temperature (qk_norm_store below), so the kernel's own arithmetic is the dot product, the cap,
 // the distance term and the softmax, all in fp32.  Options of a design: no distance term; a sink, one learned logit per
-// query head that joins the softmax's denominator without a key or a value; values that ARE the keys (rows [k: G * d]
+// query head that joins the softmax's denominator without a key or a value; kept first keys, which every later query sees
+// beside its window (0 <= i - j < window or j < keep_first); values that ARE the keys (rows [k: G * d]
 // only, read twice); a sigmoid output gate from fp32 logits laid out like the output, or one logit per head; chunks, in
 // which a query sees the keys j <= i of its own chunk only (floor(i / chunk) == floor(j / chunk), counted from the
 // sequence's first position).
@@ -14,7 +15,8 @@
 // [k: G * d | v: G * dv] in the storage type.  The norms may be absent (null weights: the projection as it is), and
 // the query may carry a temperature that grows with the position p: 1 + coef * ln(floor((p + 1) / every) + 1).
 // Further options: one root mean square over all heads of q (and of k) with a weight per number; a rotation of the first
-// rot_dims numbers of every head after the norm (dimension i with i + rot_dims / 2, angle position * inv_freq[i]); values
+// rot_dims numbers of every head after the norm (dimension i with i + rot_dims / 2, or interleaved 2i with 2i + 1, angle
+// position * inv_freq[i]); values
 // blended with another layer's values of the same token, v <- (1 - lam) v + lam v_first, before they are stored.
 //
 // window_attn_kernel: a workgroup owns TQ consecutive tokens of the packed batch and one key/value head, i.e. up to
@@ -47,6 +49,7 @@ struct QkArgs {
   const float* v_first;   // [tokens, v_first_rs] values to blend in, or null
   int64_t v_first_rs;
   const void* vmix;       // one number lam: v <- (1 - lam) v + lam v_first
+  int interleaved;        // 1: dimension 2i is rotated with 2i + 1 instead of i with i + rot_dims / 2
 };
 
 template <typename T>
@@ -115,8 +118,8 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
     auto value = [&](int e) {      // normalised, then rotated
       float x = normed(e);
       if (e < p.rot_dims) {
-        const bool first = e < half;
-        const int fi = first ? e : e - half;
+        const bool first = p.interleaved ? !(e & 1) : e < half;
+        const int fi = p.interleaved ? e >> 1 : first ? e : e - half;
         float cs, sn;
         if (trig_shared) {
           cs = s_cs[fi];
@@ -126,7 +129,8 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
           cs = cosf(a) * p.mscale;
           sn = sinf(a) * p.mscale;
         }
-        const float other = normed(first ? e + half : e - half);
+        const int pair = p.interleaved ? e ^ 1 : first ? e + half : e - half;
+        const float other = normed(pair);
         x = first ? x * cs - other * sn : x * cs + other * sn;
       }
       return x;
@@ -168,6 +172,7 @@ struct WAttnArgs {
   int64_t gate_rs;
   int gate_head;           // 1: one logit per head (head h at column h)
   int chunk;               // > 0: a query sees only the keys of its own chunk, floor(i / chunk) == floor(j / chunk)
+  int keep;                // the first `keep` keys stay visible behind the window (0: none; not together with chunk)
   int ksplit;              // SPLIT only: workgroups that share a token's keys (blockIdx.z); > 1: results go to `partial`
   float* partial;          // [tokens, H, ksplit, dv + 2]: unnormalised output, then maximum and sum
 };
@@ -225,11 +230,13 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WAttnArgs p) {
     int lo = p.window > 0 ? max(0, p0 - p.window + 1) : 0;
     if (p.chunk > 0) lo = max(lo, p0 / p.chunk * p.chunk);      // the tile's first token has the earliest chunk
     const int hi = p0 + nq - 1;
-    for (int j0 = lo; j0 <= hi; j0 += TK) {
+    // the walk is over c = base .. hi: the kept keys ahead of lo come first (c < lo: key c - base), then key c itself
+    const int base = lo - min(p.keep, lo);
+    for (int j0 = base; j0 <= hi; j0 += TK) {
       const int nk = min(TK, hi + 1 - j0);
       for (int i = tid; i < nk * (d + dv); i += 256) {
         const int j = i / (d + dv), e = i % (d + dv);
-        const int kp = j0 + j;
+        const int kp = j0 + j < lo ? j0 + j - base : j0 + j;
         const int64_t crow = (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size;
         if (e < d) sk[j * dp + e] = ld_f32<T>(cache + crow * cw + g * d + e);
         else sv[j * dv + e - d] = ld_f32<T>(cache + crow * cw + p.v_col + g * dv + e - d);
@@ -237,9 +244,9 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WAttnArgs p) {
       __syncthreads();
       for (int i = tid; i < rows * TK; i += 256) {
         const int rr = i / TK, j = i % TK;
-        const int pos = p0 + rr / R, kp = j0 + j;
+        const int pos = p0 + rr / R, kp = j0 + j < lo ? j0 + j - base : j0 + j;
         float s = -INFINITY;
-        if (j < nk && kp <= pos && (p.window <= 0 || pos - kp < p.window) && (p.chunk <= 0 || kp >= pos / p.chunk * p.chunk)) {
+        if (j < nk && kp <= pos && (p.window <= 0 || pos - kp < p.window || kp < p.keep) && (p.chunk <= 0 || kp >= pos / p.chunk * p.chunk)) {
           s = 0.0f;
           const float* qv = sq + rr * d;
           const float* kv = sk + j * dp;
@@ -315,7 +322,7 @@ constexpr size_t ma_lds_bytes(int ks, int ct, bool split) {
   return split ? 4 * (ma_stage_bytes(ks, ct) + 16 * MA_PST * 2) : ma_stage_bytes(ks, ct) + 4 * 16 * MA_PST * 2;
 }
 
-// EXT: chunks and the gate of one logit per head are compiled in; launches that use neither take the kernel without them
+// EXT: chunks, kept first keys and the gate of one logit per head are compiled in; launches that use none take the kernel without them
 template <int KS, int CT, bool SPLIT, bool EXT>
 __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
   constexpr int DK = KS * 32, KST = DK + 8, DVP = CT * 16;
@@ -395,11 +402,14 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
     const int lo_w = p.window > 0 ? max(0, p0 - p.window + 1) : 0;
     // the tile's first token has the earliest chunk
     const int lo = (EXT && p.chunk > 0) ? max(lo_w, p0 / p.chunk * p.chunk) : lo_w, hi = p0 + nq - 1;
+    // kept keys: the walk is over c = base .. hi, c < lo meaning key c - base (the kept ones ahead of the window), else key c
+    const int base = EXT ? lo - min(p.keep, lo) : lo;
+    auto key_of = [&](int c) { return EXT && c < lo ? c - base : c; };
     const int walkers = SPLIT ? 4 * p.ksplit : 1;          // wavefronts (of all workgroups) that share this token's keys
-    for (int j0 = lo + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0); j0 <= hi; j0 += walkers * MA_KEYS) {
+    for (int j0 = base + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0); j0 <= hi; j0 += walkers * MA_KEYS) {
       if (stid < MA_KEYS) {
-        const int kp = j0 + stid;
-        sRow[stid] = kp <= hi ? (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size : -1;
+        const int kp = key_of(j0 + stid);
+        sRow[stid] = j0 + stid <= hi ? (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size : -1;
       }
       sync();
       // all of a thread's loads are issued before the first LDS store: one round trip to memory per tile
@@ -437,7 +447,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
       sync();
       // keys this wavefront's rows can see: [wpos_lo - window + 1, wpos_hi]
       bool need = wave_on && j0 <= wpos_hi && (p.window <= 0 || j0 + MA_KEYS - 1 > wpos_lo - p.window);
-      if constexpr (EXT) need = need && (p.chunk <= 0 || j0 + MA_KEYS - 1 >= wpos_lo / p.chunk * p.chunk);
+      if constexpr (EXT) need = wave_on && key_of(j0) <= wpos_hi && (need || key_of(j0) < p.keep) && (p.chunk <= 0 || j0 + MA_KEYS - 1 >= wpos_lo / p.chunk * p.chunk);
       if (need) {
         f32x4 acc_s[4];
 #pragma unroll
@@ -455,12 +465,12 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
           float mt = -INFINITY;
 #pragma unroll
           for (int sub = 0; sub < 4; ++sub) {
-            const int kp = j0 + sub * 16 + lc;
+            const int kp = key_of(j0 + sub * 16 + lc);
             const int dist = pos[r] - kp;
             float sc = acc_s[sub][r];
             if (p.softcap > 0.0f) sc = p.softcap * tanhf(sc / p.softcap);
             sc -= slope[r] * (float)dist;
-            bool vis = valid[r] && dist >= 0 && (p.window <= 0 || dist < p.window);
+            bool vis = valid[r] && dist >= 0 && (p.window <= 0 || dist < p.window || (EXT && kp < p.keep));
             if constexpr (EXT) vis = vis && kp >= kmin[r];
             sc = vis ? sc : -INFINITY;
             acc_s[sub][r] = sc;
@@ -626,7 +636,7 @@ hipError_t launch_window_mfma4(const WAttnArgs& p, dim3 grid, hipStream_t s) {
 
 template <int KS, int CT, bool SPLIT>
 hipError_t launch_window_mfma3(const WAttnArgs& p, dim3 grid, hipStream_t s) {
-  if (p.chunk > 0 || (p.gate && p.gate_head)) return launch_window_mfma4<KS, CT, SPLIT, true>(p, grid, s);
+  if (p.chunk > 0 || p.keep > 0 || (p.gate && p.gate_head)) return launch_window_mfma4<KS, CT, SPLIT, true>(p, grid, s);
   return launch_window_mfma4<KS, CT, SPLIT, false>(p, grid, s);
 }
 
@@ -671,14 +681,15 @@ extern "C" int nv_qk_store(const float* proj, const void* bias, int64_t proj_row
                            void* cache, float* q_out, int64_t tokens, int heads, int kv_heads, int dim, int vdim, int dtype,
                            nv_stream_t stream) {
   return nv_qk_rotate_store(proj, bias, proj_row_stride, q_off, k_off, v_off, q_norm, k_norm, 0, temp, positions, temp_coef,
-                            temp_every, nullptr, 0, 1.0f, nullptr, 0, nullptr, scale, eps, slot_mapping, cache, q_out,
+                            temp_every, nullptr, 0, 0, 1.0f, nullptr, 0, nullptr, scale, eps, slot_mapping, cache, q_out,
                             tokens, heads, kv_heads, dim, vdim, dtype, stream);
 }
 
 extern "C" int nv_qk_rotate_store(const float* proj, const void* bias, int64_t proj_row_stride, int q_off, int k_off,
                                   int v_off, const void* q_norm, const void* k_norm, int norm_whole, const void* temp,
                                   const int64_t* positions, float temp_coef, int temp_every, const float* inv_freq,
-                                  int rot_dims, float mscale, const float* v_first, int64_t v_first_row_stride,
+                                  int rot_dims, int interleaved, float mscale, const float* v_first,
+                                  int64_t v_first_row_stride,
                                   const void* vmix, float scale, float eps, const int32_t* slot_mapping, void* cache,
                                   float* q_out, int64_t tokens, int heads, int kv_heads, int dim, int vdim, int dtype,
                                   nv_stream_t stream) {
@@ -694,7 +705,7 @@ extern "C" int nv_qk_rotate_store(const float* proj, const void* bias, int64_t p
   if (tokens == 0) return NV_OK;
   QkArgs p{proj, bias, proj_row_stride, q_off, k_off, v_off, q_norm, k_norm, temp, positions, temp_coef, temp_every,
            slot_mapping, cache, q_out, heads, kv_heads, dim, vdim, scale, eps, norm_whole, inv_freq, rot_dims, mscale,
-           v_first, v_first_row_stride, vmix};
+           v_first, v_first_row_stride, vmix, interleaved};
   NV_DISPATCH_T(dtype, qk_norm_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
   NV_CHECK_LAUNCH();
   return NV_OK;
@@ -714,14 +725,15 @@ extern "C" int nv_window_attn(const float* q, const void* cache, const int32_t* 
                               int64_t out_row_stride, int64_t tokens, int max_q, int heads, int kv_heads, int dim, int vdim,
                               int block_size, int window, float softcap, float out_scale, int dtype, nv_stream_t stream) {
   return nv_paged_softmax_attn(q, cache, block_tables, table_cols, cu_q, past_lens, seq_of_token, out, out_row_stride,
-                               tokens, max_q, heads, kv_heads, dim, vdim, block_size, window, 0, softcap, out_scale, 1, 0,
+                               tokens, max_q, heads, kv_heads, dim, vdim, block_size, window, 0, 0, softcap, out_scale, 1, 0,
                                nullptr, nullptr, 0, 0, nullptr, 0, dtype, stream);
 }
 
 extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const int32_t* block_tables, int table_cols,
                                      const int32_t* cu_q, const int32_t* past_lens, const int32_t* seq_of_token, void* out,
                                      int64_t out_row_stride, int64_t tokens, int max_q, int heads, int kv_heads, int dim,
-                                     int vdim, int block_size, int window, int chunk, float softcap, float out_scale,
+                                     int vdim, int block_size, int window, int chunk, int keep_first, float softcap,
+                                     float out_scale,
                                      int distance_term, int values_are_keys, const void* sink, const float* gate,
                                      int64_t gate_row_stride, int gate_per_head, void* workspace, size_t workspace_bytes,
                                      int dtype, nv_stream_t stream) {
@@ -730,8 +742,9 @@ extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const in
   const int cw = values_are_keys ? kv_heads * dim : kv_heads * (dim + vdim), v_col = values_are_keys ? 0 : kv_heads * dim;
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_window_attn: bad dtype %d", dtype);
   NV_CHECK_ARG(tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0 &&
-                   block_size > 0 && window >= 0 && chunk >= 0 && table_cols > 0,
+                   block_size > 0 && window >= 0 && chunk >= 0 && keep_first >= 0 && table_cols > 0,
                "nv_window_attn: bad shape");
+  NV_CHECK_ARG(chunk == 0 || keep_first == 0, "nv_window_attn: chunks and kept first keys exclude each other");
   if (tokens == 0) return NV_OK;
   const int R = heads / kv_heads;
   // bf16 caches with 16-byte-aligned heads of up to 256 numbers: the matrix-core kernel
@@ -749,7 +762,7 @@ extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const in
         ksplit = 1;
       WAttnArgs pm{q, cache, block_tables, table_cols, cu_q, past_lens, seq_of_token, out, out_row_stride, tokens, heads,
                    kv_heads, dim, vdim, block_size, window, TQm, MA_KEYS, softcap, out_scale, cw, v_col, distance_term, sink,
-                   gate, gate_row_stride, gate_per_head, chunk, ksplit, reinterpret_cast<float*>(workspace)};
+                   gate, gate_row_stride, gate_per_head, chunk, keep_first, ksplit, reinterpret_cast<float*>(workspace)};
       dim3 gridm((unsigned)((tokens + TQm - 1) / TQm), (unsigned)kv_heads, (unsigned)ksplit);
       hipStream_t st = (hipStream_t)stream;
       const hipError_t e = ks == 2 ? launch_window_mfma<2>(pm, ct, split, gridm, st)
@@ -779,7 +792,7 @@ extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const in
   const int64_t tiles = (tokens + TQ - 1) / TQ;
   WAttnArgs p{q, cache, block_tables, table_cols, cu_q, past_lens, seq_of_token, out, out_row_stride, tokens, heads,
               kv_heads, dim, vdim, block_size, window, TQ, TK, softcap, out_scale, cw, v_col, distance_term, sink, gate,
-              gate_row_stride, gate_per_head, chunk, 1, nullptr};
+              gate_row_stride, gate_per_head, chunk, keep_first, 1, nullptr};
   dim3 grid((unsigned)tiles, (unsigned)kv_heads);
   NV_DISPATCH_T(dtype, window_attn_kernel<T><<<grid, dim3(256), need(TQ, TK), (hipStream_t)stream>>>(p));
   NV_CHECK_LAUNCH();

@@ -437,10 +437,11 @@ def stage_decode_packed(packed, bs, bt_cols, g, prev_tokens=None, block_size=0):
 # Kernels of models with an fp32 residual stream (bf16 or true fp32 storage): nv_linear and its row-wise companions.
 
 EPI_NONE, EPI_GLU, EPI_SOFTCAP, EPI_ROW_GATE, EPI_ACT = 0, 1, 2, 3, 4
-ACT_SILU, ACT_GELU_TANH, ACT_XIELU, ACT_SCALE = 0, 1, 2, 3
+ACT_SILU, ACT_GELU_TANH, ACT_XIELU, ACT_SCALE, ACT_GELU_ERF = 0, 1, 2, 3, 4
 GATE_PER_NUMBER = 1  # EPI_ROW_GATE only (as ``act``): one gate logit per output number instead of one per row and batch
 GLU_CLAMPED = 2      # EPI_GLU only: g sigmoid(1.702 g) (u + 1) with g = min(gate, cap), u = clamp(up, -cap, cap)
-ROUTE_CHOSEN, ROUTE_ALL = 0, 1   # softmax over the chosen logits / over every expert, renormalised over the chosen
+# softmax over the chosen logits / over every expert, renormalised over the chosen / the sigmoid of each chosen logit
+ROUTE_CHOSEN, ROUTE_ALL, ROUTE_SIGMOID = 0, 1, 2
 
 
 def _code32(dt) -> int:
@@ -449,11 +450,12 @@ def _code32(dt) -> int:
 
 def linear(x, w, bias=None, out=None, out_dtype=None, *, rows=None, a_rows=None, batch=1, a_batch_stride=0,
            w_batch_stride=0, out_batch_stride=0, group_offsets=None, max_group_rows=None, epilogue=EPI_NONE,
-           act=ACT_SILU, gate=None, gate_stride=0, cap=0.0, n=None):
+           act=ACT_SILU, gate=None, gate_stride=0, cap=0.0, n=None, row_scale=None):
     """nv_linear.  ``x`` [M, >=K] (row stride free) in the model dtype, ``w`` [.., K] rows of the same dtype.
     Plain: w [N, K] -> out [M, N].  ``batch`` > 1: per-batch element strides select the operands (heads).
     ``group_offsets`` [batch + 1]: batch b owns output rows [off[b], off[b+1]) (experts), ``a_rows`` maps an output row to
-    its row of x, ``max_group_rows`` bounds a group.  GLU: w holds n gate rows then n up rows per batch."""
+    its row of x, ``max_group_rows`` bounds a group.  GLU: w holds n gate rows then n up rows per batch (and so does the
+    bias).  ``row_scale`` fp32 [output rows] multiplies the product ahead of bias and epilogue."""
     require_gpu(x, "linear")
     assert x.dim() == 2 and x.stride(1) == 1 and w.stride(-1) == 1 and w.dtype == x.dtype and w.is_cuda
     K = w.size(-1)
@@ -463,14 +465,17 @@ def linear(x, w, bias=None, out=None, out_dtype=None, *, rows=None, a_rows=None,
     # prefill-sized plain products of a 16-bit model go where the engine sends its other many-row products: the vendor
     # library, here with the result left in fp32
     if (epilogue in (EPI_NONE, EPI_GLU, EPI_ACT) and batch == 1 and group_offsets is None and a_rows is None
-            and (bias is None or (epilogue == EPI_ACT and (out_dtype or x.dtype) == x.dtype)) and out is None
+            and (bias is None or (epilogue != EPI_NONE and (out_dtype or x.dtype) == x.dtype)) and out is None
+            and row_scale is None
             and rows is None and x.dtype == torch.bfloat16 and (out_dtype or x.dtype) in (torch.float32, torch.bfloat16)
             and w.dim() == 2 and w.is_contiguous() and x.stride(0) % 8 == 0 and use_many_rows_path(M, K, n) and K % 8 == 0
             and n % 8 == 0 and x.data_ptr() % 16 == 0):
         if epilogue == EPI_GLU:      # [gate | up] rows from the library, activation and product in one pass over them
             y = _linear_many_rows(x, w, M, 2 * n, K, torch.float32)
             out = torch.empty(M, n, dtype=out_dtype or x.dtype, device=x.device)
-            check(lib().nv_act_mul_f32(ptr(y), ptr(out), M, n, act, cap, _code32(out.dtype), stream()), "nv_act_mul_f32")
+            assert bias is None or (bias.dtype == x.dtype and bias.numel() == 2 * n and bias.is_contiguous())
+            check(lib().nv_bias_act_mul_f32(ptr(y), ptr(bias), ptr(out), M, n, act, cap, _code32(out.dtype), stream()),
+                  "nv_bias_act_mul_f32")
             return out
         if epilogue == EPI_ACT:      # the element-wise function in one pass over the library's fp32 result
             y = _linear_many_rows(x, w, M, n, K, torch.float32)
@@ -490,16 +495,20 @@ def linear(x, w, bias=None, out=None, out_dtype=None, *, rows=None, a_rows=None,
     assert out.stride(-1) == 1 and out.dtype == out_dtype
     if bias is not None:
         assert bias.dtype == x.dtype and bias.is_contiguous()
+        assert bias.numel() >= n * (2 if epilogue == EPI_GLU else 1)
+    if row_scale is not None:
+        assert row_scale.dtype == torch.float32 and row_scale.is_contiguous() and row_scale.numel() == M
     if gate is not None:
         assert gate.dtype == torch.float32
     if group_offsets is not None:
         assert group_offsets.dtype == torch.int32 and group_offsets.numel() == batch + 1
     if a_rows is not None:
         assert a_rows.dtype == torch.int32
-    check(lib().nv_linear(ptr(x), x.stride(0), ptr(a_rows), ptr(w), w.stride(-2), ptr(bias), ptr(out), out.stride(0),
-                          _code32(out_dtype), grid_rows, n, K, batch, a_batch_stride, w_batch_stride, out_batch_stride,
-                          n if bias is not None and batch > 1 else 0, ptr(group_offsets), epilogue, act, ptr(gate),
-                          gate_stride, cap, _code32(x.dtype), stream()), "nv_linear")
+    bias_stride = n * (2 if epilogue == EPI_GLU else 1) if bias is not None and batch > 1 else 0
+    check(lib().nv_linear_scaled(ptr(x), x.stride(0), ptr(a_rows), ptr(w), w.stride(-2), ptr(bias), ptr(out), out.stride(0),
+                                 _code32(out_dtype), grid_rows, n, K, batch, a_batch_stride, w_batch_stride,
+                                 out_batch_stride, bias_stride, ptr(group_offsets), epilogue, act, ptr(gate), gate_stride,
+                                 cap, ptr(row_scale), _code32(x.dtype), stream()), "nv_linear_scaled")
     return out
 
 
@@ -549,6 +558,39 @@ def rms_norm_f32(x, w, eps, out=None):
     out = torch.empty(x.shape, dtype=w.dtype, device=x.device) if out is None else out
     check(lib().nv_rmsnorm_f32(ptr(x), x.stride(0), ptr(w), ptr(out), out.stride(0), x.size(0), x.size(1), eps,
                                _code32(w.dtype), stream()), "nv_rmsnorm_f32")
+    return out
+
+
+def sandwich_norm(x, y, w_post, w_pre, eps, y_bias=None, rows_idx=None, slot_of=None, weights=None, last_gate=None,
+                  shared=None, shared_gate=None):
+    """fp32 residual rows ``x`` [T, n] take a sublayer's result through its output norm, x += rms_norm(v) * w_post, in
+    place; -> rms_norm(x) * w_pre in the weights' dtype (``w_pre`` None: nothing).  v = ``y`` [T, n] + ``y_bias``, or with
+    ``slot_of`` int32 [T, C] the sum of f_i * y[slot_of[t, i]] (expert rows; f = ``weights`` [T, C] or 1, the last one
+    sigmoid(``last_gate`` [T]) when given) plus ``shared`` [T, n] times sigmoid(``shared_gate`` [T]).  ``y`` None: the norm
+    alone.  ``rows_idx``: only these rows are normed, and ``x`` is left as it is."""
+    require_gpu(x, "sandwich_norm")
+    T, n = x.shape
+    assert x.dtype == torch.float32 and x.is_contiguous()
+    w = w_pre if w_pre is not None else w_post
+    for v in (w_post, w_pre, y_bias):
+        assert v is None or (v.dtype == w.dtype and v.numel() == n and v.is_contiguous())
+    if y is not None:
+        assert y.dtype == torch.float32 and y.stride(1) == 1 and y.size(1) == n and (slot_of is not None or y.size(0) == T)
+    if slot_of is not None:
+        assert slot_of.dtype == torch.int32 and slot_of.is_contiguous() and slot_of.size(0) == T
+        assert weights is None or (weights.dtype == torch.float32 and weights.is_contiguous()
+                                   and weights.shape == slot_of.shape)
+    for g in (last_gate, shared_gate):
+        assert g is None or (g.dtype == torch.float32 and g.dim() == 1 and g.numel() == T)
+    assert shared is None or (shared.dtype == torch.float32 and shared.is_contiguous() and shared.shape == (T, n))
+    assert rows_idx is None or rows_idx.dtype == torch.int32
+    rows = T if rows_idx is None else rows_idx.numel()
+    out = torch.empty(rows, n, dtype=w.dtype, device=x.device) if w_pre is not None else None
+    check(lib().nv_sandwich_norm(ptr(x), ptr(y), y.stride(0) if y is not None else 0, ptr(y_bias), ptr(w_post), ptr(w_pre),
+                                 ptr(out), n, ptr(rows_idx), ptr(slot_of), slot_of.size(1) if slot_of is not None else 0,
+                                 ptr(weights), ptr(last_gate), last_gate.stride(0) if last_gate is not None else 0,
+                                 ptr(shared), ptr(shared_gate), shared_gate.stride(0) if shared_gate is not None else 0,
+                                 rows, n, eps, _code32(w.dtype), stream()), "nv_sandwich_norm")
     return out
 
 
@@ -754,6 +796,25 @@ def moe_combine(y, slot_of, weights, shared=None, shared_gate=None, out=None):
     return out
 
 
+def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False):
+    """Routing and ordering of fp32 router logits [T, >= experts].  With ``shared`` every token's last choice is expert
+    number ``experts`` (weight 1): C = top + 1 choices and experts + 1 groups, else C = top.
+    -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C], sorted row of every
+    choice int32 [T, C], the routed choices' weights fp32 [T, top])."""
+    require_gpu(logits, "moe_plan")
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.size(1) >= experts
+    T, dev, C = logits.size(0), logits.device, top + int(shared)
+    idx = torch.empty(T, top, dtype=torch.int32, device=dev)
+    weights = torch.empty(T, top, dtype=torch.float32, device=dev)
+    offsets = torch.empty(experts + int(shared) + 1, dtype=torch.int32, device=dev)
+    sorted_token = torch.empty(T * C, dtype=torch.int32, device=dev)
+    sorted_weight = torch.empty(T * C, dtype=torch.float32, device=dev)
+    slot_of = torch.empty(T, C, dtype=torch.int32, device=dev)
+    check(lib().nv_moe_plan(ptr(logits), logits.stride(0), T, experts, top, mode, int(shared), ptr(idx), ptr(weights),
+                            ptr(offsets), ptr(sorted_token), ptr(sorted_weight), ptr(slot_of), stream()), "nv_moe_plan")
+    return offsets, sorted_token, sorted_weight, slot_of, weights
+
+
 # ---- residual streams, token shift, shaped-score attention, recurrences with state slots ----
 def embed_sinusoid(ids, positions, table, inv_freq, streams, out=None):
     """fp32 streams [T, streams, width], each table[id] + (sin, cos) pairs of position * inv_freq (float64 [ceil(width/2)])."""
@@ -860,12 +921,13 @@ def window_attn(q, cache, block_tables, cu_q, past_lens, seq_of_token, max_q, he
 
 
 def qk_rotate_store(proj, offsets, positions, scale, slot_mapping, cache, heads, kv_heads, dim, vdim, *, q_norm=None,
-                    k_norm=None, eps=0.0, inv_freq=None, rot_dims=0, mscale=1.0, v_first=None, vmix=None, bias=None):
+                    k_norm=None, eps=0.0, inv_freq=None, rot_dims=0, interleaved=False, mscale=1.0, v_first=None,
+                    vmix=None, bias=None):
     """fp32 projections [T, *] with q | k | v at ``offsets`` -> fp32 queries [T, heads * dim] times ``scale``; keys and
     values go to cache rows [G * dim | G * vdim] of ``slot_mapping``.  ``q_norm`` [heads * dim] / ``k_norm``
     [kv_heads * dim]: one RMS norm over all of a token's query numbers (and all of its key numbers) with a weight per
     number.  ``rot_dims``: the first rot_dims numbers of every head turn by position * inv_freq[i], i with
-    i + rot_dims / 2.  ``v_first`` fp32 [T, G * vdim] (a column slice is fine): the stored values are
+    i + rot_dims / 2 (``interleaved``: 2i with 2i + 1).  ``v_first`` fp32 [T, G * vdim] (a column slice is fine): the stored values are
     (1 - vmix) v + vmix v_first."""
     require_gpu(proj, "qk_rotate_store")
     T = proj.size(0)
@@ -889,7 +951,7 @@ def qk_rotate_store(proj, offsets, positions, scale, slot_mapping, cache, heads,
     q = torch.empty(T, heads * dim, dtype=torch.float32, device=proj.device)
     check(lib().nv_qk_rotate_store(ptr(proj), ptr(bias), proj.stride(0), q_off, k_off, v_off, ptr(q_norm), ptr(k_norm),
                                    int(q_norm is not None), None, ptr(positions), 0.0, 0, ptr(inv_freq), int(rot_dims),
-                                   float(mscale), ptr(v_first), v_first.stride(0) if v_first is not None else 0,
+                                   int(interleaved), float(mscale), ptr(v_first), v_first.stride(0) if v_first is not None else 0,
                                    ptr(vmix) if v_first is not None else None, scale, eps, ptr(slot_mapping), ptr(cache),
                                    ptr(q), T, heads, kv_heads, dim, vdim, _code32(cache.dtype), stream()),
           "nv_qk_rotate_store")
@@ -919,11 +981,12 @@ def qk_store(proj, offsets, positions, scale, slot_mapping, cache, heads, kv_hea
 
 def paged_softmax_attn(q, cache, block_tables, cu_q, past_lens, seq_of_token, max_q, heads, kv_heads, dim, vdim, block_size,
                        out, window=0, softcap=0.0, out_scale=1.0, distance_term=False, values_are_keys=False, sink=None,
-                       gate=None, chunk=0, gate_per_head=False):
+                       gate=None, chunk=0, gate_per_head=False, keep_first=0):
     """window_attn with its options spelled out: no distance term unless asked for, cache rows that hold keys only and
     serve as values too, a sink logit per head in the denominator, a sigmoid gate (fp32 logits laid out like the
     output, or with ``gate_per_head`` one per head) folded into the store, and ``chunk`` > 0: a query sees the keys
-    of its own chunk of the sequence only."""
+    of its own chunk of the sequence only; ``keep_first`` > 0: the first keys of the sequence stay visible
+    beside the window."""
     require_gpu(q, "paged_softmax_attn")
     T = q.size(0)
     assert q.dtype == torch.float32 and q.is_contiguous() and q.size(1) == heads * dim and cache.is_contiguous()
@@ -940,7 +1003,7 @@ def paged_softmax_attn(q, cache, block_tables, cu_q, past_lens, seq_of_token, ma
     ws = workspace(nbytes, q.device, "paged_softmax_attn") if nbytes else None
     check(lib().nv_paged_softmax_attn(ptr(q), ptr(cache), ptr(block_tables), block_tables.size(1), ptr(cu_q),
                                       ptr(past_lens), ptr(seq_of_token), ptr(out), out.stride(0), T, max_q, heads, kv_heads,
-                                      dim, vdim, block_size, window, int(chunk), float(softcap or 0.0), out_scale,
+                                      dim, vdim, block_size, window, int(chunk), int(keep_first), float(softcap or 0.0), out_scale,
                                       int(distance_term), int(values_are_keys), ptr(sink), ptr(gate),
                                       gate.stride(0) if gate is not None else 0, int(gate_per_head), ptr(ws), nbytes,
                                       _code32(cache.dtype), stream()),

@@ -11,7 +11,8 @@ from torch import nn
 from byox_vllm_amd import kernels
 from byox_vllm_amd.layers.linear import DenseLinear
 
-UNARY = {"silu": kernels.ACT_SILU, "gelu_tanh": kernels.ACT_GELU_TANH, "xielu": kernels.ACT_XIELU}
+UNARY = {"silu": kernels.ACT_SILU, "gelu_tanh": kernels.ACT_GELU_TANH, "xielu": kernels.ACT_XIELU,
+         "gelu_erf": kernels.ACT_GELU_ERF}
 
 
 class UnaryMLP(nn.Module):

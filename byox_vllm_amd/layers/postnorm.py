@@ -7,7 +7,14 @@ taps - 1 inputs are a request's state, layers/conv.py).  The update of the resid
 the PREVIOUS sublayer's pending result into the fp32 residual (one launch: gate, norm, scaled add, and a copy of the new
 rows in the model dtype for the gate's product), then hands out the sublayer's input and the gate logits; the caller
 runs f and passes (y, gate logits, this module) on as the next pending result.  All of it is fp32
-(csrc/rowops.hip: nv_gated_postnorm_add); eps sits inside the root."""
+(csrc/rowops.hip: nv_gated_postnorm_add); eps sits inside the root.
+
+``SandwichNorm`` is the pair of norms around a sublayer that is normed on both sides:
+
+    x <- x + rms_norm(f(rms_norm(x) * w_pre)) * w_post
+
+Its update is deferred the same way: ``begin`` takes the PREVIOUS sublayer's result through that sublayer's output norm
+into the residual and norms the new rows for this one, in one launch (csrc/rowops.hip: nv_sandwich_norm)."""
 
 import torch
 from torch import nn
@@ -59,3 +66,25 @@ class GatedPostNorm(nn.Module):
             h = conv(x, want_f32=False, want_t=True)[1] if conv is not None else rows
         logits = kernels.linear(rows, self.gate.weight.data, out_dtype=torch.float32) if self.gate is not None else None
         return h, logits
+
+
+class SandwichNorm(nn.Module):
+    def __init__(self, width: int, eps: float, final: bool = False):
+        """``final``: the norm behind the last sublayer, which has no output norm of its own."""
+        super().__init__()
+        self.eps = float(eps)
+        self.pre = nn.Parameter(torch.ones(width), requires_grad=False)
+        self.post = None if final else nn.Parameter(torch.ones(width), requires_grad=False)
+
+    def begin(self, x: torch.Tensor, pending, rows_idx=None) -> torch.Tensor:
+        """``pending`` = (the previous sublayer's result as keywords of kernels.sandwich_norm, its SandwichNorm) or None.
+        -> this sublayer's input in the model dtype (of the rows ``rows_idx`` only, if given: ``x`` then stays as it is)."""
+        result, norm = pending if pending is not None else ({"y": None}, None)
+        return kernels.sandwich_norm(x, w_post=norm.post.data if norm is not None else None, w_pre=self.pre.data, eps=self.eps,
+                                     rows_idx=rows_idx, **result)
+
+    @staticmethod
+    def settle(x: torch.Tensor, pending) -> None:
+        """The pending result joins ``x`` (nothing is normed for a next sublayer)."""
+        result, norm = pending
+        kernels.sandwich_norm(x, w_post=norm.post.data, w_pre=None, eps=norm.eps, **result)

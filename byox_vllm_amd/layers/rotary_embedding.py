@@ -46,12 +46,22 @@ def scaled_inv_freq(dims: int, base: float, scaling: dict | None = None) -> tupl
     to the dimension index dims * ln(original / (2 pi t)) / (2 ln base); between the indices of ``fast`` (floor, at
     least 0) and ``slow`` (ceil, at most dims - 1) a linear ramp blends the plain frequency (ramp 0, fast-rotating
     dimensions keep theirs) into the frequency divided by ``factor`` (ramp 1); the magnitude factor is
-    0.1 ln(factor) + 1.  The rotation itself (angle = position * frequency in fp32) runs inside the kernels."""
+    0.1 ln(factor) + 1.
+
+    With scaling by wavelength {factor, original, low, high} (Llama 3.1): a pair whose wavelength 2 pi / f is below
+    original / high keeps f, above original / low it gets f / factor, and between the two the pair blends both linearly in
+    s = (original / wavelength - low) / (high - low); the magnitude factor is 1.  The rotation itself (angle = position * frequency in fp32) runs inside the kernels."""
     import math
     i = torch.arange(dims // 2, dtype=torch.float64)
     freq = torch.as_tensor(float(base), dtype=torch.float64) ** (-2.0 * i / dims)
     magnitude = 1.0
-    if scaling:
+    if scaling and "low" in scaling:
+        factor, original, low, high = (float(scaling[k]) for k in ("factor", "original", "low", "high"))
+        wavelength = 2.0 * math.pi / freq
+        s = (original / wavelength - low) / (high - low) if high != low else torch.ones_like(freq)
+        blend = (1.0 - s) * freq / factor + s * freq
+        freq = torch.where(wavelength < original / high, freq, torch.where(wavelength > original / low, freq / factor, blend))
+    elif scaling:
         factor, original = float(scaling["factor"]), float(scaling["original"])
 
         def index_of(turns: float) -> float:

@@ -343,13 +343,22 @@ int nv_gemm_lt_f32out(const void* x, int64_t x_row_stride, const void* w_rowmajo
  *                3 row gate: out *= sigmoid(epi_ptr[m * epi_row_stride + b]), one logit per row and batch element
  *                (act 0), or one per output number, epi_ptr[m * epi_row_stride + b * N + n] (act 1);
  *                4 element-wise function chosen by act: 0 SiLU, 1 tanh-form GELU, 2 xIELU (a z^2 + z/2 for z > 0,
- *                b (exp(z) - 1 - z) + z/2 otherwise, with a = epi_ptr[0], b = epi_ptr[1]), 3 out *= epi_const;
+ *                b (exp(z) - 1 - z) + z/2 otherwise, with a = epi_ptr[0], b = epi_ptr[1]), 3 out *= epi_const, 4 erf-form
+ *                GELU;
+ *   bias         [N] per batch element; of the gated unit [2 N], the gate rows' then the up rows';
  *   out_dtype    NV_BF16 or NV_F32, independent of the operands' dtype. */
 int nv_linear(const void* a, int64_t a_row_stride, const int32_t* a_rows, const void* w, int64_t w_row_stride,
               const void* bias, void* out, int64_t out_row_stride, int out_dtype, int64_t M, int N, int K, int batch,
               int64_t a_batch_stride, int64_t w_batch_stride, int64_t out_batch_stride, int64_t bias_batch_stride,
               const int32_t* group_offsets, int epilogue, int act, const float* epi_ptr, int64_t epi_row_stride,
               float epi_const, int dtype, nv_stream_t stream);
+/* ... with a factor per output row (fp32, may be null) that multiplies the product ahead of bias and epilogue: f(s W a)
+ * = f(W (s a)), so a mixture that weighs its experts' INPUT needs no scaled copy of the rows. */
+int nv_linear_scaled(const void* a, int64_t a_row_stride, const int32_t* a_rows, const void* w, int64_t w_row_stride,
+                     const void* bias, void* out, int64_t out_row_stride, int out_dtype, int64_t M, int N, int K, int batch,
+                     int64_t a_batch_stride, int64_t w_batch_stride, int64_t out_batch_stride, int64_t bias_batch_stride,
+                     const int32_t* group_offsets, int epilogue, int act, const float* epi_ptr, int64_t epi_row_stride,
+                     float epi_const, const float* row_scale, int dtype, nv_stream_t stream);
 
 /* out[t] = table[ids[t]] * scale as fp32 rows (the residual stream's first value). */
 int nv_embed_scale(const int64_t* ids, const void* table, float* out, int64_t tokens, int width, int64_t vocab,
@@ -385,6 +394,20 @@ int nv_gated_postnorm_add_conv(float* x, const float* y, int64_t y_row_stride, c
                                int taps, float* conv_state, const int32_t* state_slots, const int32_t* past_lens,
                                void* conv_out, int64_t conv_out_row_stride, int dtype, nv_stream_t stream);
 
+/* A sublayer normed before and after: row t of the fp32 residual takes the previous sublayer's result through ITS output
+ * norm, and the next sublayer's input norm reads the sum, in one launch:
+ *   v = y + y_bias,  x += v / sqrt(mean(v^2) + eps) * w_post,  out = x / sqrt(mean(x^2) + eps) * w_pre (storage type).
+ * y null: x as it is; w_post null: x += v; w_pre / out null: the residual only.  slot_of [rows, choices] (may be null):
+ * v is the sum over i of f_i * y[slot_of[t][i]] (rows of a mixture's experts; f_i = weights[t * choices + i], 1 when
+ * weights is null; with last_gate the last choice has f = sigmoid(last_gate[t * last_gate_stride])) plus, when given,
+ * shared[t] * sigmoid(shared_gate[t * shared_gate_stride]).  rows_idx: output row i is made from row rows_idx[i] of x and
+ * of y's arrays, and x is left as it is. */
+int nv_sandwich_norm(float* x, const float* y, int64_t y_row_stride, const void* y_bias, const void* w_post,
+                     const void* w_pre, void* out, int64_t out_row_stride, const int32_t* rows_idx, const int32_t* slot_of,
+                     int choices, const float* weights, const float* last_gate, int64_t last_gate_stride,
+                     const float* shared, const float* shared_gate, int64_t shared_gate_stride, int64_t rows, int n,
+                     float eps, int dtype, nv_stream_t stream);
+
 /* RMS norm of fp32 rows: out = x / sqrt(mean(x^2) + eps) * w, rounded to the storage type. */
 int nv_rmsnorm_f32(const float* x, int64_t x_row_stride, const void* w, void* out, int64_t out_row_stride, int64_t rows,
                    int n, float eps, int dtype, nv_stream_t stream);
@@ -397,6 +420,9 @@ int nv_act_f32(const float* y, void* out, int64_t total, int act, const float* p
 int nv_bias_act_f32(const float* y, const void* bias, int n, void* out, int64_t total, int act, const float* params,
                     float c, int dtype, nv_stream_t stream);
 int nv_act_mul_f32(const float* y, void* out, int64_t rows, int n, int act, float c, int dtype, nv_stream_t stream);
+/* ... of y + bias, bias [2 n] in the storage type (null: none). */
+int nv_bias_act_mul_f32(const float* y, const void* bias, void* out, int64_t rows, int n, int act, float c, int dtype,
+                        nv_stream_t stream);
 
 /* Sampler over fp32 logits: temperature 0 -> argmax (lowest index on ties), else Gumbel-max with noise hashed from
  * (seed, row, column). */
@@ -458,11 +484,18 @@ int nv_latent_attn(const float* qa, const void* cache, const int32_t* block_tabl
                    int rot_dim, int block_size, int window, float scale, int dtype, nv_stream_t stream);
 
 /* Mixture of experts (csrc/moe.hip): routing, ordering by expert, weighted combination.  nv_moe_route mode 0: softmax
- * over the chosen logits; 1: softmax over all experts, chosen scores divided by (their sum + 1e-20).  nv_moe_combine
+ * over the chosen logits; 1: softmax over all experts, chosen scores divided by (their sum + 1e-20); 2: the sigmoid of
+ * the chosen logits as it is.  nv_moe_plan routes and orders: weights as nv_moe_route's [tokens, top]; with shared = 1
+ * every token also has choice `top`, expert number `experts` with weight 1, so the arrays cover top + shared choices per
+ * token and experts + shared groups; sorted_weight (may be null) is the weight of every sorted row.  Short steps take one
+ * launch.  nv_moe_combine
  * adds `shared` times sigmoid(shared_gate) per token, or `shared` as it is when shared_gate is null. */
 int nv_moe_route(const float* logits, int64_t row_stride, int32_t* idx, float* weights, int64_t tokens, int experts,
                  int top, int mode, nv_stream_t stream);
 int nv_moe_sort(const int32_t* idx, int64_t tokens, int experts, int top, int32_t* offsets, int32_t* sorted_token,
+                int32_t* slot_of, nv_stream_t stream);
+int nv_moe_plan(const float* logits, int64_t row_stride, int64_t tokens, int experts, int top, int mode, int shared,
+                int32_t* idx, float* weights, int32_t* offsets, int32_t* sorted_token, float* sorted_weight,
                 int32_t* slot_of, nv_stream_t stream);
 int nv_moe_combine(const float* y, const int32_t* slot_of, const float* weights, int top, const float* shared,
                    const float* shared_gate, int64_t shared_gate_stride, float* out, int64_t tokens, int width,
@@ -514,11 +547,12 @@ int nv_window_attn(const float* q, const void* cache, const int32_t* block_table
  *   values (vdim == dim); sink [heads] (storage type, may be null) adds exp(sink[h]) to the softmax's denominator; gate
  *   (fp32 [tokens, gate_row_stride], head h at h * vdim, or with gate_per_head one logit per head at column h; may be
  *   null) multiplies the output by its sigmoid; chunk > 0 restricts a query to the keys of its own chunk,
- *   floor(i / chunk) == floor(j / chunk), positions counted from the sequence's start.
+ *   floor(i / chunk) == floor(j / chunk), positions counted from the sequence's start; keep_first > 0 (not together with
+ *   chunk): the sequence's first keep_first keys stay visible to every later query beside its window.
  * nv_qk_rotate_store: nv_qk_store with three more options.  norm_whole: one root mean square over all heads * dim query
  *   numbers (and all kv_heads * dim key numbers), weights [heads * dim] and [kv_heads * dim].  rot_dims > 0: after the
- *   norm the first rot_dims numbers of every query and key head are rotated, dimension i with i + rot_dims / 2, by the
- *   angle positions[t] * inv_freq[i], cosine and sine times mscale.  v_first (fp32 [tokens, v_first_row_stride], may be
+ *   norm the first rot_dims numbers of every query and key head are rotated, dimension i with i + rot_dims / 2 (interleaved:
+ *   2i with 2i + 1), by the angle positions[t] * inv_freq[i], cosine and sine times mscale.  v_first (fp32 [tokens, v_first_row_stride], may be
  *   null): the stored values are (1 - lam) v + lam v_first with lam = vmix[0] (storage type). */
 int nv_qk_store(const float* proj, const void* bias, int64_t proj_row_stride, int q_off, int k_off, int v_off,
                 const void* q_norm, const void* k_norm, const void* temp, const int64_t* positions, float temp_coef,
@@ -527,12 +561,12 @@ int nv_qk_store(const float* proj, const void* bias, int64_t proj_row_stride, in
 int nv_paged_softmax_attn(const float* q, const void* cache, const int32_t* block_tables, int table_cols,
                           const int32_t* cu_q, const int32_t* past_lens, const int32_t* seq_of_token, void* out,
                           int64_t out_row_stride, int64_t tokens, int max_q, int heads, int kv_heads, int dim, int vdim,
-                          int block_size, int window, int chunk, float softcap, float out_scale, int distance_term,
-                          int values_are_keys, const void* sink, const float* gate, int64_t gate_row_stride,
+                          int block_size, int window, int chunk, int keep_first, float softcap, float out_scale,
+                          int distance_term, int values_are_keys, const void* sink, const float* gate, int64_t gate_row_stride,
                           int gate_per_head, void* workspace, size_t workspace_bytes, int dtype, nv_stream_t stream);
 int nv_qk_rotate_store(const float* proj, const void* bias, int64_t proj_row_stride, int q_off, int k_off, int v_off,
                        const void* q_norm, const void* k_norm, int norm_whole, const void* temp, const int64_t* positions,
-                       float temp_coef, int temp_every, const float* inv_freq, int rot_dims, float mscale,
+                       float temp_coef, int temp_every, const float* inv_freq, int rot_dims, int interleaved, float mscale,
                        const float* v_first, int64_t v_first_row_stride, const void* vmix, float scale, float eps,
                        const int32_t* slot_mapping, void* cache, float* q_out, int64_t tokens, int heads, int kv_heads,
                        int dim, int vdim, int dtype, nv_stream_t stream);
