@@ -230,13 +230,13 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WAttnArgs p) {
     int lo = p.window > 0 ? max(0, p0 - p.window + 1) : 0;
     if (p.chunk > 0) lo = max(lo, p0 / p.chunk * p.chunk);      // the tile's first token has the earliest chunk
     const int hi = p0 + nq - 1;
-    // the walk is over c = base .. hi: the kept keys ahead of lo come first (c < lo: key c - base), then key c itself
-    const int base = lo - min(p.keep, lo);
-    for (int j0 = base; j0 <= hi; j0 += TK) {
+    // the walk is over c = c_first .. hi: the kept keys ahead of lo come first (c < lo: key c - c_first), then key c itself
+    const int c_first = lo - min(p.keep, lo);
+    for (int j0 = c_first; j0 <= hi; j0 += TK) {
       const int nk = min(TK, hi + 1 - j0);
       for (int i = tid; i < nk * (d + dv); i += 256) {
         const int j = i / (d + dv), e = i % (d + dv);
-        const int kp = j0 + j < lo ? j0 + j - base : j0 + j;
+        const int kp = j0 + j < lo ? j0 + j - c_first : j0 + j;
         const int64_t crow = (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size;
         if (e < d) sk[j * dp + e] = ld_f32<T>(cache + crow * cw + g * d + e);
         else sv[j * dv + e - d] = ld_f32<T>(cache + crow * cw + p.v_col + g * dv + e - d);
@@ -244,9 +244,10 @@ __global__ __launch_bounds__(256) void window_attn_kernel(WAttnArgs p) {
       __syncthreads();
       for (int i = tid; i < rows * TK; i += 256) {
         const int rr = i / TK, j = i % TK;
-        const int pos = p0 + rr / R, kp = j0 + j < lo ? j0 + j - base : j0 + j;
+        const int pos = p0 + rr / R, kp = j0 + j < lo ? j0 + j - c_first : j0 + j;
         float s = -INFINITY;
-        if (j < nk && kp <= pos && (p.window <= 0 || pos - kp < p.window || kp < p.keep) && (p.chunk <= 0 || kp >= pos / p.chunk * p.chunk)) {
+        if (j < nk && kp <= pos && (p.window <= 0 || pos - kp < p.window || kp < p.keep) &&
+            (p.chunk <= 0 || kp >= pos / p.chunk * p.chunk)) {
           s = 0.0f;
           const float* qv = sq + rr * d;
           const float* kv = sk + j * dp;
@@ -322,7 +323,8 @@ constexpr size_t ma_lds_bytes(int ks, int ct, bool split) {
   return split ? 4 * (ma_stage_bytes(ks, ct) + 16 * MA_PST * 2) : ma_stage_bytes(ks, ct) + 4 * 16 * MA_PST * 2;
 }
 
-// EXT: chunks, kept first keys and the gate of one logit per head are compiled in; launches that use none take the kernel without them
+// EXT: chunks, kept first keys and the gate of one logit per head are compiled in; launches that use none of them take
+// the kernel without
 template <int KS, int CT, bool SPLIT, bool EXT>
 __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
   constexpr int DK = KS * 32, KST = DK + 8, DVP = CT * 16;
@@ -402,11 +404,11 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
     const int lo_w = p.window > 0 ? max(0, p0 - p.window + 1) : 0;
     // the tile's first token has the earliest chunk
     const int lo = (EXT && p.chunk > 0) ? max(lo_w, p0 / p.chunk * p.chunk) : lo_w, hi = p0 + nq - 1;
-    // kept keys: the walk is over c = base .. hi, c < lo meaning key c - base (the kept ones ahead of the window), else key c
-    const int base = EXT ? lo - min(p.keep, lo) : lo;
-    auto key_of = [&](int c) { return EXT && c < lo ? c - base : c; };
+    // kept keys: the walk is over c = c_first .. hi; c < lo means key c - c_first (those ahead of the window), else key c
+    const int c_first = EXT ? lo - min(p.keep, lo) : lo;
+    auto key_of = [&](int c) { return EXT && c < lo ? c - c_first : c; };
     const int walkers = SPLIT ? 4 * p.ksplit : 1;          // wavefronts (of all workgroups) that share this token's keys
-    for (int j0 = base + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0); j0 <= hi; j0 += walkers * MA_KEYS) {
+    for (int j0 = c_first + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0); j0 <= hi; j0 += walkers * MA_KEYS) {
       if (stid < MA_KEYS) {
         const int kp = key_of(j0 + stid);
         sRow[stid] = j0 + stid <= hi ? (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size : -1;
@@ -447,7 +449,9 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
       sync();
       // keys this wavefront's rows can see: [wpos_lo - window + 1, wpos_hi]
       bool need = wave_on && j0 <= wpos_hi && (p.window <= 0 || j0 + MA_KEYS - 1 > wpos_lo - p.window);
-      if constexpr (EXT) need = wave_on && key_of(j0) <= wpos_hi && (need || key_of(j0) < p.keep) && (p.chunk <= 0 || j0 + MA_KEYS - 1 >= wpos_lo / p.chunk * p.chunk);
+      if constexpr (EXT)
+        need = wave_on && key_of(j0) <= wpos_hi && (need || key_of(j0) < p.keep) &&
+               (p.chunk <= 0 || j0 + MA_KEYS - 1 >= wpos_lo / p.chunk * p.chunk);
       if (need) {
         f32x4 acc_s[4];
 #pragma unroll
