@@ -282,8 +282,8 @@ def run_generate_workload(args):
     print(json.dumps(line), flush=True)
 
 
-# --arch-compare: the Rurutar, Nonetar, Zamusun and Kikelorn designs beside the dense Qwen3 decoder (and beside each other) at equal
-# width, depth, active feed-forward size and vocabulary, both through LLM.generate: prefill and decode tokens/s.
+# --arch-compare: the Rurutar, Nonetar, Zamusun, Kikelorn and Vasonex designs beside the dense Qwen3 decoder (and beside each
+# other) at equal width, depth, active feed-forward size and vocabulary, both through LLM.generate: prefill and decode tokens/s.
 # name: (width, layers, prompts, prompt length, decoded tokens)
 ARCH_COMPARE_SIZES = {
     "w1024": (1024, 8, 8, 2048, 64),
@@ -391,6 +391,25 @@ def kikelorn_bench_config(width: int, layers: int, vocab: int = 32000):
     return kikelorn_config(raw, dtype=torch.bfloat16)
 
 
+def vasonex_bench_config(width: int, layers: int, vocab: int = 32000):
+    """A Vasonex configuration with the proportions of a real model's layers: attention with two query heads per key head
+    of 128, a window of 512 tokens beside 16 kept ones, a quarter of each head rotated; dense gated feed-forwards of the
+    dense comparator's size in turn with mixtures of 16 experts, two per token, beside a shared one, whose active
+    parameters equal it; the last two layers use the weights of the two before them."""
+    from byox_vllm_amd.models.vasonex import vasonex_config
+    heads = width // 128
+    mixer = {"heads": heads, "kv_heads": max(1, heads // 2), "dim": 128, "vdim": 128, "scale": 128 ** -0.5,
+             "mask": {"size": 512, "keep_first": 16},
+             "rot": {"base": 500000.0, "dims": 32, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}}
+    moe = {"kind": "moe", "router": {"experts": 16, "top": 2}, "expert": {"ff": 3 * width // 2}, "shared": {"ff": 3 * width // 2}}
+    specs = [{"type": "attention", "mixer": json.loads(json.dumps(mixer)),
+              "mlp": dict(moe) if i % 2 else {"kind": "dense", "ff": 3 * width}} for i in range(layers)]
+    for i in range(max(layers - 2, 4), layers):
+        specs[i]["weights_of"] = i - 2
+    raw = {"architecture": "Vasonex", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": specs}
+    return vasonex_config(raw, dtype=torch.bfloat16)
+
+
 def run_arch_compare(args):
     from byox_vllm_amd import LLM, SamplingParams
     from byox_vllm_amd.config import qwen2_config
@@ -398,7 +417,7 @@ def run_arch_compare(args):
     random.seed(0)
     results = []
     designs = {"rurutar": rurutar_bench_config, "nonetar": nonetar_bench_config, "zamusun": zamusun_bench_config,
-               "kikelorn": kikelorn_bench_config}
+               "kikelorn": kikelorn_bench_config, "vasonex": vasonex_bench_config}
     chosen = [d for d in args.arch_designs.split(",") if d]
     assert chosen and all(d in designs for d in chosen), f"--arch-designs: a subset of {sorted(designs)}"
     for name, (width, layers, num, plen, decoded) in ARCH_COMPARE_SIZES.items():
@@ -523,7 +542,7 @@ def main():
                     help="instead of the decode benchmark: prefill and decode tokens/s of the designs named by --arch-designs "
                          "beside the dense Qwen3 decoder at equal size (one GPU, LLM.generate)")
     ap.add_argument("--arch-designs", default="rurutar",
-                    help="--arch-compare: the designs to run beside the dense decoder, comma-separated (rurutar, nonetar, zamusun, kikelorn)")
+                    help="--arch-compare: the designs to run beside the dense decoder, comma-separated (rurutar, nonetar, zamusun, kikelorn, vasonex)")
     ap.add_argument("--arch-sizes", default="", help="--arch-compare: comma-separated subset of " + ",".join(ARCH_COMPARE_SIZES))
     args = ap.parse_args()
     if args.arch_compare:

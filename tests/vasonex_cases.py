@@ -4,6 +4,7 @@ windows shorter and longer than a page, kept tokens fewer and more than a window
 rotations over all, part and none of a head, one expert and several per token, shared experts of the experts' size, of
 another size and absent, layers without a feed-forward, weights used by one to three layers, also through a chain."""
 
+import contextlib
 import copy
 
 import torch
@@ -144,8 +145,14 @@ class Engine:
         self.runner = ModelRunner(self.config, 0, None)
         self.scheduler = Scheduler(self.config)
         self.block_size = block_size
+        self.rows, self.moe_calls = [], 0        # (request, position) of the step's rows; mixtures run so far in it
+        self.forced = None                       # request -> experts its tokens are to take (ForcedRoutes)
 
     def replay(self, requests: dict, schedule: list):
+        with ForcedRoutes(self, self.forced) if self.forced is not None else contextlib.nullcontext():
+            return self._replay(requests, schedule)
+
+    def _replay(self, requests: dict, schedule: list):
         """requests: name -> token list; schedule: steps of [(name, count)].  Logits of every position, per request.
         A request ends (and gives back pages and slot) with the step that brings its last token."""
         from byox_vllm_amd.engine.sequence import Sequence
@@ -161,6 +168,8 @@ class Engine:
                     live[name].extend_tokens(piece)
                 plan.append((live[name], count))
                 at[name] += count
+            self.rows = [(name, at[name] - count + i) for name, count in step for i in range(count)]
+            self.moe_calls = 0
             self.scheduler.commit(plan)
             logits = self.runner.run_portions(plan, want=[list(range(c)) for _, c in plan]).cpu()
             self.scheduler.advance(plan, [None] * len(plan))
@@ -171,6 +180,48 @@ class Engine:
                 if at[name] == len(requests[name]):
                     self.scheduler.finish(live.pop(name))
         return {n: torch.cat(v) for n, v in out.items()}
+
+
+class ForcedRoutes:
+    """While active, the engine's routers choose the experts the oracle chose (their scores stay the engine's own): a
+    router logit of random weights can lie inside the rounding of its 16-bit input, and a token that takes another expert
+    is off by much more than rounding.  ``chosen``: request -> per mixture run in order, the experts of every token."""
+
+    def __init__(self, engine, chosen: dict):
+        self.engine, self.chosen = engine, chosen
+
+    def __enter__(self):
+        from byox_vllm_amd import kernels
+        plan = self.plan = kernels.moe_plan
+
+        def forced(logits, experts, top, *rest, **kw):
+            call = self.engine.moe_calls
+            self.engine.moe_calls += 1
+            allowed = torch.zeros(logits.size(0), logits.size(1), dtype=torch.bool)
+            allowed[:, experts:] = True
+            for i, (name, pos) in enumerate(self.engine.rows):
+                allowed[i, self.chosen[name][call][pos]] = True
+            return plan(torch.where(allowed.to(logits.device), logits, logits - 1000.0), experts, top, *rest, **kw)
+        kernels.moe_plan = forced
+
+    def __exit__(self, *_):
+        from byox_vllm_amd import kernels
+        kernels.moe_plan = self.plan
+
+
+def forward_with_routes(tokens, weights, cfg):
+    """The oracle's logits and the experts its routers chose, per mixture run [T, top]."""
+    chosen, route = [], O.route
+
+    def recording(z, top):
+        idx, w = route(z, top)
+        chosen.append(idx)
+        return idx, w
+    O.route = recording
+    try:
+        return O.forward(tokens, weights, cfg), chosen
+    finally:
+        O.route = route
 
 
 def row_errors(got: torch.Tensor, want: torch.Tensor) -> torch.Tensor:
