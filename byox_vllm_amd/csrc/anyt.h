@@ -17,6 +17,27 @@ template <typename T> __device__ __forceinline__ float round_to(float v);
 template <> __device__ __forceinline__ float round_to<float>(float v) { return v; }
 template <> __device__ __forceinline__ float round_to<bf16_t>(float v) { return (float)(bf16_t)v; }
 
+// four consecutive numbers per access: 16 bytes of fp32, 8 of bf16
+template <typename T> struct Pack4;
+template <> struct Pack4<float> {
+  typedef f32x4 type;
+  static __device__ __forceinline__ f32x4 widen(const f32x4& v) { return v; }
+  static __device__ __forceinline__ f32x4 narrow(const f32x4& v) { return v; }
+};
+template <> struct Pack4<bf16_t> {
+  typedef uint2 type;
+  static __device__ __forceinline__ f32x4 widen(const uint2& v) {
+    return f32x4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
+                 __uint_as_float(v.y & 0xffff0000u)};
+  }
+  static __device__ __forceinline__ uint2 narrow(const f32x4& v) {
+    union { bf16_t h[4]; uint2 u; } r;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) r.h[i] = (bf16_t)v[i];
+    return r.u;
+  }
+};
+
 __device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu_f32(float z) { return z / (1.0f + expf(-z)); }
 __device__ __forceinline__ float gelu_tanh_f32(float z) {

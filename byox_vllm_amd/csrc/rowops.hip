@@ -54,26 +54,6 @@ __global__ __launch_bounds__(256) void rmsnorm_f32_kernel(const float* __restric
 // Post-norm residual with a gate: x[t] += mult * (g / sqrt(mean(g^2) + eps)) * w, g = (y[t] + y_bias) * sigmoid(gate[t] +
 // gate_bias) (no gate: g = y + y_bias; y_bias is the bias a producing product left to its consumer, or null); the new
 // row is also written in the storage type for the products that read the residual.  Without y the row is only copied.
-template <typename T> struct Pack4;
-template <> struct Pack4<float> {
-  typedef f32x4 type;
-  static __device__ __forceinline__ f32x4 widen(const f32x4& v) { return v; }
-  static __device__ __forceinline__ f32x4 narrow(const f32x4& v) { return v; }
-};
-template <> struct Pack4<bf16_t> {
-  typedef uint2 type;
-  static __device__ __forceinline__ f32x4 widen(const uint2& v) {
-    return f32x4{__uint_as_float(v.x << 16), __uint_as_float(v.x & 0xffff0000u), __uint_as_float(v.y << 16),
-                 __uint_as_float(v.y & 0xffff0000u)};
-  }
-  static __device__ __forceinline__ uint2 narrow(const f32x4& v) {
-    union { bf16_t h[4]; uint2 u; } r;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) r.h[i] = (bf16_t)v[i];
-    return r.u;
-  }
-};
-
 // The input convolution of the NEXT sublayer, for steps in which row t is request t's only token: every earlier row a
 // tap reads is in the request's slot, so the launch that makes the new residual row also hands out x + conv(x) and moves
 // the slot on (csrc/scan.hip has the general form).

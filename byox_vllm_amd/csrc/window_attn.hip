@@ -19,6 +19,8 @@
 // position * inv_freq[i]); values
 // blended with another layer's values of the same token, v <- (1 - lam) v + lam v_first, before they are stored.
 //
+// qk_pairs_store_kernel: the same where a number depends on itself and its neighbour only.
+//
 // window_attn_kernel: a workgroup owns TQ consecutive tokens of the packed batch and one key/value head, i.e. up to
 // TQ * (H / G) query rows that read the same keys; tokens of different requests inside the tile are served one request
 // after the other.  Keys go through LDS in tiles of TK rows; online softmax per row.
@@ -148,6 +150,51 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
       float x = row[p.v_off + e] + (bias ? ld_f32<T>(bias + p.v_off + e) : 0.0f);
       if (p.v_first) x = (1.0f - lam) * x + lam * p.v_first[t * p.v_first_rs + e];
       st_f32<T>(crow + p.G * p.d + e, x);
+    }
+  }
+}
+
+// The case without norms, temperatures, biases and blended values whose rotation (if any) is interleaved: every output
+// depends on a pair of neighbouring inputs, so a thread takes four consecutive numbers of q | k | v per access.
+template <typename T>
+__global__ __launch_bounds__(256) void qk_pairs_store_kernel(QkArgs p) {
+  typedef typename Pack4<T>::type P;
+  __shared__ float s_cs[128], s_sn[128];
+  const int64_t t = blockIdx.x;
+  const float* row = p.proj + t * p.proj_rs;
+  const int64_t slot = p.slot_mapping[t];
+  const int nq = p.H * p.d, nk = p.G * p.d, nv = p.G * p.dv, half = p.rot_dims / 2;
+  T* crow = slot >= 0 ? reinterpret_cast<T*>(p.cache) + slot * (nk + nv) : nullptr;
+  if (half > 0) {
+    const float pos = (float)p.positions[t];
+    for (int i = threadIdx.x; i < half; i += 256) {
+      const float a = pos * p.inv_freq[i];
+      s_cs[i] = cosf(a) * p.mscale;
+      s_sn[i] = sinf(a) * p.mscale;
+    }
+    __syncthreads();
+  }
+  for (int c = threadIdx.x * 4; c < nq + nk + nv; c += 1024) {
+    const bool is_q = c < nq, is_v = c >= nq + nk;
+    const int rel = is_q ? c : is_v ? c - nq - nk : c - nq;
+    f32x4 x = *reinterpret_cast<const f32x4*>(row + (is_q ? p.q_off : is_v ? p.v_off : p.k_off) + rel);
+    if (!is_v) {
+      const int e = rel % p.d;
+#pragma unroll
+      for (int j = 0; j < 4; j += 2) {
+        if (e + j < p.rot_dims) {
+          const float cs = s_cs[(e + j) >> 1], sn = s_sn[(e + j) >> 1], u = x[j], v = x[j + 1];
+          x[j] = u * cs - v * sn;
+          x[j + 1] = v * cs + u * sn;
+        }
+      }
+    }
+    if (is_q) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) x[j] *= p.scale;
+      *reinterpret_cast<f32x4*>(p.q_out + t * nq + rel) = x;
+    } else if (crow) {
+      *reinterpret_cast<P*>(crow + (is_v ? nk : 0) + rel) = Pack4<T>::narrow(x);
     }
   }
 }
@@ -587,6 +634,174 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
   }
 }
 
+// ---- one token per request, few query heads per key head (bf16 cache) ----
+// A decoded token's R query rows are far too few for a matrix-core tile to pay for its staging, so the keys stay in
+// registers: LPK lanes share a key, eight numbers (16 bytes) each, a wavefront reads KPW = 64 / LPK keys per access and U
+// such accesses of keys and of values are in flight before the first is used.  Scores are reduced over the LPK lanes; every
+// group of LPK lanes keeps its own running maximum, sum and weighted values, which meet by shuffles, then in LDS.  All of it
+// is fp32.  Workgroups (blockIdx.z) and their wavefronts take every 4 * ksplit-th batch of KPW * U keys.
+template <int LPK, int RP, int U>
+__global__ __launch_bounds__(256) void window_attn_rows_kernel(WAttnArgs p) {
+  constexpr int KPW = 64 / LPK, KB = KPW * U;
+  static_assert(KB <= 64, "one lane looks up one key of a batch");
+  __shared__ float part[4][RP][LPK * 8 + 2];
+  const int R = p.H / p.G, d = p.d, dv = p.dv;
+  const int64_t t = blockIdx.x;
+  const int g = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int li = lane % LPK, sub = lane / LPK;
+  const int b = p.seq_of[t];
+  const int pos = p.past[b] + (int)(t - p.cu_q[b]);
+  const int32_t* table = p.tables + (int64_t)b * p.table_cols;
+  const bf16_t* cache = reinterpret_cast<const bf16_t*>(p.cache);
+  const int cw = p.cw;
+  const bool k_on = li * 8 < d, v_on = li * 8 < dv;
+  float q[RP][8], acc[RP][8], m[RP], l[RP];
+#pragma unroll
+  for (int r = 0; r < RP; ++r) {
+    const float* qr = p.q + (t * p.H + g * R + r) * d + li * 8;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      q[r][e] = (r < R && k_on) ? qr[e] : 0.0f;
+      acc[r][e] = 0.0f;
+    }
+    m[r] = -INFINITY;
+    l[r] = 0.0f;
+  }
+  int lo = p.window > 0 ? max(0, pos - p.window + 1) : 0;
+  if (p.chunk > 0) lo = max(lo, pos / p.chunk * p.chunk);
+  const int c_first = lo - min(p.keep, lo);               // kept keys ahead of the window, as in the other kernels
+  for (int c0 = c_first + ((int)blockIdx.z * 4 + wv) * KB; c0 <= pos; c0 += 4 * p.ksplit * KB) {
+    int64_t row_of = -1;
+    {
+      const int c = c0 + lane;
+      if (lane < KB && c <= pos) {
+        const int kp = c < lo ? c - c_first : c;
+        row_of = (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size;
+      }
+    }
+    u32x4 kr[U], vr[U];
+    bool seen[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int64_t row = __shfl(row_of, u * KPW + sub, 64);
+      seen[u] = row >= 0;
+      kr[u] = vr[u] = u32x4{0u, 0u, 0u, 0u};
+      if (seen[u] && k_on) kr[u] = *reinterpret_cast<const u32x4*>(cache + row * cw + g * d + li * 8);
+      if (seen[u] && v_on) vr[u] = *reinterpret_cast<const u32x4*>(cache + row * cw + p.v_col + g * dv + li * 8);
+    }
+    float s[RP][U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+#pragma unroll
+      for (int r = 0; r < RP; ++r) {
+        float a = 0.0f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w)
+          a += q[r][2 * w] * lo_f32<bf16_t>(kr[u][w]) + q[r][2 * w + 1] * hi_f32<bf16_t>(kr[u][w]);
+        s[r][u] = a;
+      }
+    }
+#pragma unroll
+    for (int o = 1; o < LPK; o <<= 1) {
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int r = 0; r < RP; ++r) s[r][u] += __shfl_xor(s[r][u], o, 64);
+    }
+#pragma unroll
+    for (int r = 0; r < RP; ++r) {
+      const float slope = p.slope_on ? exp2f(-8.0f * (float)(g * R + r + 1) / (float)p.H) : 0.0f;
+      float mt = m[r];
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const int c = c0 + u * KPW + sub, kp = c < lo ? c - c_first : c;
+        float a = s[r][u];
+        if (p.softcap > 0.0f) a = p.softcap * tanhf(a / p.softcap);
+        a -= slope * (float)(pos - kp);
+        s[r][u] = seen[u] ? a : -INFINITY;
+        mt = fmaxf(mt, s[r][u]);
+      }
+      const float corr = mt == -INFINITY ? 1.0f : __expf(m[r] - mt);
+      m[r] = mt;
+      l[r] *= corr;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[r][e] *= corr;
+#pragma unroll
+      for (int u = 0; u < U; ++u) {
+        const float e_ = s[r][u] == -INFINITY ? 0.0f : __expf(s[r][u] - mt);
+        l[r] += e_;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+          acc[r][2 * w] += e_ * lo_f32<bf16_t>(vr[u][w]);
+          acc[r][2 * w + 1] += e_ * hi_f32<bf16_t>(vr[u][w]);
+        }
+      }
+    }
+  }
+  // the KPW groups of a wavefront
+#pragma unroll
+  for (int o = LPK; o < 64; o <<= 1) {
+#pragma unroll
+    for (int r = 0; r < RP; ++r) {
+      const float m2 = __shfl_xor(m[r], o, 64), l2 = __shfl_xor(l[r], o, 64);
+      const float mt = fmaxf(m[r], m2);
+      const float f1 = m[r] == -INFINITY ? 0.0f : __expf(m[r] - mt), f2 = m2 == -INFINITY ? 0.0f : __expf(m2 - mt);
+      l[r] = l[r] * f1 + l2 * f2;
+      m[r] = mt;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[r][e] = acc[r][e] * f1 + __shfl_xor(acc[r][e], o, 64) * f2;
+    }
+  }
+  if (sub == 0) {
+#pragma unroll
+    for (int r = 0; r < RP; ++r) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) part[wv][r][li * 8 + e] = acc[r][e];
+      if (li == 0) {
+        part[wv][r][LPK * 8] = m[r];
+        part[wv][r][LPK * 8 + 1] = l[r];
+      }
+    }
+  }
+  __syncthreads();
+  const bf16_t* sink = reinterpret_cast<const bf16_t*>(p.sink);
+  bf16_t* out = reinterpret_cast<bf16_t*>(p.out);
+  for (int i = tid; i < R * dv; i += 256) {
+    const int r = i / dv, e = i % dv, h = g * R + r;
+    float mt = -INFINITY, sum = 0.0f, o = 0.0f;
+#pragma unroll
+    for (int w = 0; w < 4; ++w) mt = fmaxf(mt, part[w][r][LPK * 8]);
+#pragma unroll
+    for (int w = 0; w < 4; ++w) {
+      const float mw = part[w][r][LPK * 8];
+      const float f = mw == -INFINITY ? 0.0f : __expf(mw - mt);
+      sum += part[w][r][LPK * 8 + 1] * f;
+      o += part[w][r][e] * f;
+    }
+    if (p.ksplit > 1) {
+      float* dst = p.partial + ((t * p.H + h) * p.ksplit + blockIdx.z) * (dv + 2);
+      dst[e] = o;
+      if (e == 0) {
+        dst[dv] = mt;
+        dst[dv + 1] = sum;
+      }
+      continue;
+    }
+    float f, den;
+    close_softmax(mt, sum, sink != nullptr, sink ? ld_f32<bf16_t>(sink + h) : 0.0f, f, den);
+    float v = o * f * p.out_scale / den;
+    if (p.gate) v *= sigmoid_f32(p.gate[t * p.gate_rs + (p.gate_head ? h : h * dv + e)]);
+    out[t * p.out_rs + h * dv + e] = (bf16_t)v;
+  }
+}
+
+template <int LPK>
+void launch_window_rows(const WAttnArgs& p, int R, dim3 grid, hipStream_t s) {
+  if (R == 1) window_attn_rows_kernel<LPK, 1, LPK == 8 ? 4 : 8><<<grid, dim3(256), 0, s>>>(p);
+  else if (R == 2) window_attn_rows_kernel<LPK, 2, LPK == 8 ? 4 : 8><<<grid, dim3(256), 0, s>>>(p);
+  else window_attn_rows_kernel<LPK, 4, 4><<<grid, dim3(256), 0, s>>>(p);
+}
+
 // joins the shares of the ksplit workgroups that walked one token's keys: one wavefront per (token, head)
 __global__ __launch_bounds__(256) void window_attn_join_kernel(WAttnArgs p) {
   const int64_t row = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
@@ -707,10 +922,17 @@ extern "C" int nv_qk_rotate_store(const float* proj, const void* bias, int64_t p
                "nv_qk_store: a rotation over %d of %d numbers needs positions and frequencies", rot_dims, dim);
   NV_CHECK_ARG(!v_first || (vmix && vdim > 0), "nv_qk_store: blending values needs its weight");
   if (tokens == 0) return NV_OK;
+  auto al = [](const void* q, size_t n) { return (uintptr_t)q % n == 0; };
+  const bool pairs = !q_norm && !temp && !bias && !v_first && temp_every == 0 && (rot_dims == 0 || (interleaved && rot_dims <= 256)) &&
+                     dim % 4 == 0 && vdim % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 &&
+                     proj_row_stride % 4 == 0 && al(proj, 16) && al(q_out, 16) && al(cache, 16);
   QkArgs p{proj, bias, proj_row_stride, q_off, k_off, v_off, q_norm, k_norm, temp, positions, temp_coef, temp_every,
            slot_mapping, cache, q_out, heads, kv_heads, dim, vdim, scale, eps, norm_whole, inv_freq, rot_dims, mscale,
            v_first, v_first_row_stride, vmix, interleaved};
-  NV_DISPATCH_T(dtype, qk_norm_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
+  if (pairs)
+    NV_DISPATCH_T(dtype, qk_pairs_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
+  else
+    NV_DISPATCH_T(dtype, qk_norm_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
@@ -759,9 +981,10 @@ extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const in
     if (ma_lds_bytes(ks, ct, false) <= 160 * 1024) {
       // one token per request: the wavefronts split the window (where four staging areas fit the LDS)
       const bool split = max_q <= 1 && R <= 16 && ma_lds_bytes(ks, ct, true) <= 156 * 1024;
+      const bool rows = max_q <= 1 && R <= 4 && getenv("NV_WINDOW_ATTN_ROWS_OFF") == nullptr;   // keys in registers
       const int TQm = max_q <= 1 ? 1 : 64 / R;
       // ... and with few requests several workgroups do, when the caller brought room for their shares
-      int ksplit = split ? window_attn_key_splits(tokens, kv_heads) : 1;
+      int ksplit = split || rows ? window_attn_key_splits(tokens, kv_heads) : 1;
       if (ksplit > 1 && (!workspace || workspace_bytes < (size_t)tokens * heads * ksplit * (vdim + 2) * sizeof(float)))
         ksplit = 1;
       WAttnArgs pm{q, cache, block_tables, table_cols, cu_q, past_lens, seq_of_token, out, out_row_stride, tokens, heads,
@@ -769,7 +992,11 @@ extern "C" int nv_paged_softmax_attn(const float* q, const void* cache, const in
                    gate, gate_row_stride, gate_per_head, chunk, keep_first, ksplit, reinterpret_cast<float*>(workspace)};
       dim3 gridm((unsigned)((tokens + TQm - 1) / TQm), (unsigned)kv_heads, (unsigned)ksplit);
       hipStream_t st = (hipStream_t)stream;
-      const hipError_t e = ks == 2 ? launch_window_mfma<2>(pm, ct, split, gridm, st)
+      const int wide = dim > vdim ? dim : vdim;
+      if (rows && wide <= 64) launch_window_rows<8>(pm, R, gridm, st);
+      else if (rows && wide <= 128) launch_window_rows<16>(pm, R, gridm, st);
+      else if (rows) launch_window_rows<32>(pm, R, gridm, st);
+      const hipError_t e = rows ? hipGetLastError() : ks == 2 ? launch_window_mfma<2>(pm, ct, split, gridm, st)
                            : ks == 4 ? launch_window_mfma<4>(pm, ct, split, gridm, st)
                                      : launch_window_mfma<8>(pm, ct, split, gridm, st);
       if (e != hipSuccess) {

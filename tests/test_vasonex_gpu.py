@@ -323,7 +323,8 @@ def _plain(proj, offs, H, G, d, dv, scale, mask, gate=None):
     return out.reshape(T, H * dv)
 
 
-GEOMETRIES = [(6, 2, 16, 24, 16), (1, 1, 20, 12, 16), (8, 1, 128, 40, 64), (4, 4, 72, 16, 16), (3, 1, 10, 6, 32)]
+GEOMETRIES = [(6, 2, 16, 24, 16), (1, 1, 20, 12, 16), (8, 1, 128, 40, 64), (4, 4, 72, 16, 16), (3, 1, 10, 6, 32), (4, 2, 136, 200, 16),
+              (12, 3, 24, 64, 32), (2, 2, 256, 256, 64)]
 MASKS = [(12, 3), (16, 0), (5, 30), (1, 1), (64, 17), (0, 4), (200, 200), (33, 70)]
 
 
