@@ -111,6 +111,28 @@ __device__ __forceinline__ void rows_pair32(float x, float& lower, float& upper)
   upper = __uint_as_float(b);
 }
 
+// Sum / maximum over aligned groups of N = 8 or 16 lanes on the VALU (DPP: neighbours, pairs, the mirrored half row, the
+// mirrored row), without the LDS crossbar a __shfl_xor goes through; every lane gets the same bits.
+template <int CTRL> __device__ __forceinline__ float dpp_f32(float x) {
+  return __uint_as_float((uint32_t)__builtin_amdgcn_update_dpp(0, (int)__float_as_uint(x), CTRL, 0xf, 0xf, false));
+}
+template <int N> __device__ __forceinline__ float lanes_sum(float v) {
+  static_assert(N == 8 || N == 16, "lanes_sum: groups of 8 or 16 lanes");
+  v += dpp_f32<0xB1>(v);         // quad_perm [1, 0, 3, 2]
+  v += dpp_f32<0x4E>(v);         // quad_perm [2, 3, 0, 1]
+  v += dpp_f32<0x141>(v);        // row_half_mirror
+  if constexpr (N == 16) v += dpp_f32<0x140>(v);   // row_mirror
+  return v;
+}
+template <int N> __device__ __forceinline__ float lanes_max(float v) {
+  static_assert(N == 8 || N == 16, "lanes_max: groups of 8 or 16 lanes");
+  v = fmaxf(v, dpp_f32<0xB1>(v));
+  v = fmaxf(v, dpp_f32<0x4E>(v));
+  v = fmaxf(v, dpp_f32<0x141>(v));
+  if constexpr (N == 16) v = fmaxf(v, dpp_f32<0x140>(v));
+  return v;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

@@ -373,11 +373,11 @@ constexpr size_t ma_lds_bytes(int ks, int ct, bool split) {
 // EXT: chunks, kept first keys and the gate of one logit per head are compiled in; launches that use none of them take
 // the kernel without
 template <int KS, int CT, bool SPLIT, bool EXT>
-__global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
+__global__ __launch_bounds__(256, (!SPLIT && KS <= 4 && CT <= 8) ? 2 : 1) void window_attn_mfma_kernel(WAttnArgs p) {
   constexpr int DK = KS * 32, KST = DK + 8, DVP = CT * 16;
   constexpr int STAGE = (int)(ma_stage_bytes(KS, CT) / 2);                 // bf16 elements of one staging area
   extern __shared__ u32x4 lds_raw[];
-  __shared__ int64_t sRowAll[SPLIT ? 4 : 1][MA_KEYS];
+  __shared__ int64_t sRowAll[SPLIT ? 4 : 1][2][MA_KEYS];
   const int R = p.H / p.G, d = p.d, dv = p.dv;
   const int g = blockIdx.y;
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
@@ -386,7 +386,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
   bf16_t* sK = base + (SPLIT ? wv * STAGE : 0);              // [64][KST]
   bf16_t* sVt = sK + MA_KEYS * KST;                          // [DVP][MA_VST]
   bf16_t* sPw = base + (SPLIT ? 4 : 1) * STAGE + wv * 16 * MA_PST;   // [16][MA_PST] of this wavefront
-  int64_t* sRow = sRowAll[SPLIT ? wv : 0];
+  int64_t (*sRows)[MA_KEYS] = sRowAll[SPLIT ? wv : 0];     // cache rows of this tile's keys and of the next one's
   constexpr int ST = SPLIT ? 64 : 256;                                    // threads that stage a tile together
   constexpr int NKC = MA_KEYS * (DK / 8) / ST, NVC = MA_KEYS * (DVP / 8) / ST;   // 16-byte pieces per thread
   const int stid = SPLIT ? lane : tid;
@@ -455,12 +455,17 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
     const int c_first = EXT ? lo - min(p.keep, lo) : lo;
     auto key_of = [&](int c) { return EXT && c < lo ? c - c_first : c; };
     const int walkers = SPLIT ? 4 * p.ksplit : 1;          // wavefronts (of all workgroups) that share this token's keys
-    for (int j0 = c_first + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0); j0 <= hi; j0 += walkers * MA_KEYS) {
-      if (stid < MA_KEYS) {
-        const int kp = key_of(j0 + stid);
-        sRow[stid] = j0 + stid <= hi ? (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size : -1;
-      }
-      sync();
+    const int j_first = c_first + (SPLIT ? ((int)blockIdx.z * 4 + wv) * MA_KEYS : 0);
+    auto row_of = [&](int c) {
+      const int kp = key_of(c);
+      return c <= hi ? (int64_t)table[kp / p.block_size] * p.block_size + kp % p.block_size : (int64_t)-1;
+    };
+    int turn = 0;
+    if (stid < MA_KEYS) sRows[0][stid] = row_of(j_first + stid);
+    sync();
+    for (int j0 = j_first; j0 <= hi; j0 += walkers * MA_KEYS) {
+      const int64_t* sRow = sRows[turn];
+      turn ^= 1;
       // all of a thread's loads are issued before the first LDS store: one round trip to memory per tile
       u32x4 kreg[NKC], vreg[NVC];
 #pragma unroll
@@ -478,6 +483,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
         if (row >= 0 && part * 8 < dv)
           vreg[i] = *reinterpret_cast<const u32x4*>(cache + row * cw + p.v_col + g * dv + part * 8);
       }
+      if (stid < MA_KEYS) sRows[turn][stid] = row_of(j0 + walkers * MA_KEYS + stid);      // its table entry is on the way with them
 #pragma unroll
       for (int i = 0; i < NKC; ++i) {
         const int c = stid + i * ST, key = c / (DK / 8), part = c % (DK / 8);
@@ -527,8 +533,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
             acc_s[sub][r] = sc;
             mt = fmaxf(mt, sc);
           }
-#pragma unroll
-          for (int o = 1; o < 16; o <<= 1) mt = fmaxf(mt, __shfl_xor(mt, o, 64));
+          mt = lanes_max<16>(mt);
           const float m_new = fmaxf(m_run[r], mt);
           corr[r] = m_new == -INFINITY ? 1.0f : __expf(m_run[r] - m_new);
           float sum = 0.0f;
@@ -539,8 +544,7 @@ __global__ __launch_bounds__(256) void window_attn_mfma_kernel(WAttnArgs p) {
             sum += e;
             sPw[(lg * 4 + r) * MA_PST + sub * 16 + lc] = (bf16_t)e;
           }
-#pragma unroll
-          for (int o = 1; o < 16; o <<= 1) sum += __shfl_xor(sum, o, 64);
+          sum = lanes_sum<16>(sum);
           l_run[r] = l_run[r] * corr[r] + sum;
           m_run[r] = m_new;
         }
@@ -702,11 +706,12 @@ __global__ __launch_bounds__(256) void window_attn_rows_kernel(WAttnArgs p) {
       }
     }
 #pragma unroll
-    for (int o = 1; o < LPK; o <<= 1) {
+    for (int u = 0; u < U; ++u) {
 #pragma unroll
-      for (int u = 0; u < U; ++u)
-#pragma unroll
-        for (int r = 0; r < RP; ++r) s[r][u] += __shfl_xor(s[r][u], o, 64);
+      for (int r = 0; r < RP; ++r) {
+        s[r][u] = lanes_sum<LPK == 8 ? 8 : 16>(s[r][u]);
+        if constexpr (LPK == 32) s[r][u] += __shfl_xor(s[r][u], 16, 64);
+      }
     }
 #pragma unroll
     for (int r = 0; r < RP; ++r) {
