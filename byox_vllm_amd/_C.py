@@ -77,7 +77,9 @@ _PROTOS = {
     "nv_gated_postnorm_add_conv": (_i, [_p, _p, _i64, _p, _p, _i64, _p, _p, _p, _i64, _i64, _i, _f, _f, _p, _i, _p, _p, _p,
                                         _p, _i64, _i, _p]),
     "nv_bias_act_f32": (_i, [_p, _p, _i, _p, _i64, _i, _p, _f, _i, _p]),
-    "nv_sandwich_norm": (_i, [_p, _p, _i64, _p, _p, _p, _p, _i64, _p, _p, _i, _p, _p, _i64, _p, _p, _i64, _i64, _i, _f, _i, _p]),
+    "nv_sandwich_norm": (_i, [_p, _p, _i64, _p, _p, _p, _p, _i64, _p, _p, _i, _p, _p, _i64, _p, _p, _i64, _p, _p,
+                              _i64, _i, _f, _i, _p]),
+    "nv_rotation_table": (_i, [_p, _p, _p, _i64, _i, _p]),
     "nv_rmsnorm_f32": (_i, [_p, _i64, _p, _p, _i64, _i64, _i, _f, _i, _p]),
     "nv_act_mul_f32": (_i, [_p, _p, _i64, _i, _i, _f, _i, _p]),
     "nv_bias_act_mul_f32": (_i, [_p, _p, _p, _i64, _i, _i, _f, _i, _p]),
@@ -86,7 +88,7 @@ _PROTOS = {
     "nv_gla_recurrent": (_i, [_p, _i64, _i, _i, _i, _i, _p, _i64, _p, _p, _p, _p, _p, _p, _i, _i, _i, _i, _f, _f, _f, _i, _p]),
     "nv_matrix_memory_state_size": (_i64, [_i, _i, _i]),
     "nv_matrix_memory": (_i, [_p, _i64, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _i, _f, _f,
-                              _i, _p]),
+                              _p, _i, _f, _i, _p]),
     "nv_residual_pair": (_i, [_p, _p, _i64, _p, _p, _i64, _i, _i, _p]),
     "nv_latent_kv_store": (_i, [_p, _i64, _p, _p, _p, _f, _p, _p, _i64, _i, _i, _i, _i, _f, _i, _p]),
     "nv_latent_q_rope": (_i, [_p, _i64, _p, _p, _f, _p, _i64, _i, _i, _i, _i, _i, _i, _i, _p]),
@@ -98,12 +100,12 @@ _PROTOS = {
     "nv_latent_expand": (_i, [_p, _p, _p, _i64, _i, _i, _i, _i, _i, _i, _p]),
     "nv_moe_route": (_i, [_p, _i64, _p, _p, _i64, _i, _i, _i, _p]),
     "nv_moe_sort": (_i, [_p, _i64, _i, _i, _p, _p, _p, _p]),
-    "nv_moe_plan": (_i, [_p, _i64, _i64, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p]),
+    "nv_moe_plan": (_i, [_p, _i64, _i64, _i, _i, _i, _i, _i, _p, _i, _i, _f, _p, _p, _p, _p, _p, _p, _p, _p]),
     "nv_moe_combine": (_i, [_p, _p, _p, _i, _p, _p, _i64, _p, _i64, _i, _p]),
     "nv_embed_sinusoid": (_i, [_p, _p, _p, _p, _p, _i64, _i, _i, _i64, _i, _p]),
     "nv_hc_norm": (_i, [_p, _i, _i, _p, _i64, _p, _p, _p, _i, _f, _p, _p, _i64, _i, _i64, _i, _p]),
     "nv_token_shift": (_i, [_p, _p, _p, _p, _p, _p, _p, _p, _i64, _i, _i, _p]),
-    "nv_group_rmsnorm_f32": (_i, [_p, _i64, _p, _p, _i64, _i64, _i, _i, _f, _p, _i64, _i, _p]),
+    "nv_group_rmsnorm_f32": (_i, [_p, _i64, _p, _p, _i64, _i64, _i, _i, _f, _p, _i64, _i, _i, _p]),
     "nv_qk_norm_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _p, _f, _f, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
     "nv_window_attn": (_i, [_p, _p, _p, _i, _p, _p, _p, _p, _i64, _i64, _i, _i, _i, _i, _i, _i, _i, _f, _f, _i, _p]),
     "nv_qk_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _p, _p, _f, _i, _f, _f, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
@@ -111,6 +113,9 @@ _PROTOS = {
                                    _i, _p, _p, _i64, _i, _p, _sz, _i, _p]),
     "nv_qk_rotate_store": (_i, [_p, _p, _i64, _i, _i, _i, _p, _p, _i, _p, _p, _f, _i, _p, _i, _i, _f, _p, _i64, _p, _f, _f, _p,
                                 _p, _p, _i64, _i, _i, _i, _i, _i, _p]),
+    "nv_qk_conv_store_ok": (_i, [_p, _i64, _i, _i, _i, _p, _p, _p, _i, _i, _i]),
+    "nv_qk_conv_store": (_i, [_p, _i64, _i, _i, _i, _p, _i, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _i, _f, _f,
+                              _i, _p]),
     "nv_paged_softmax_attn_workspace_bytes": (_sz, [_i64, _i, _i, _i, _i]),
     "nv_causal_conv": (_i, [_p, _p, _i64, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i, _i, _i, _p]),
     "nv_causal_conv_batch": (_i, [_p, _p, _i64, _p, _p, _p, _p, _p, _p, _p, _p, _i64, _p, _i64, _i64, _i, _i, _i, _i, _i,

@@ -1,8 +1,8 @@
 // Matrix memories with one decay per head and token: a per-head state S [dim, vdim] in fp32,
 //   S_t = keep_t S_(t-1) + take_t k_t v_t^T,   o_t = S_t^T q_t,
 // in two forms.
-//   MEM_CONST  (lightning attention): keep_t = decay[h], a constant of the head, take_t = 1; q, k, v may pass through
-//              SiLU first; o_t leaves as it is.
+//   MEM_CONST  (lightning attention, retention): keep_t = decay[h], a constant of the head, take_t = 1; q, k, v may pass
+//              through SiLU first, q and k may be rotated by their position; o_t leaves as it is.
 //   MEM_EXPGATE (the matrix memory of xLSTM): log gates i_t = cap tanh(zi / cap) and f_t = logsigmoid(cap tanh(zf / cap))
 //              from one logit each per head, a running maximum m_t = max(f_t + m_(t-1), i_t) that starts at 0,
 //              keep_t = exp(f_t + m_(t-1) - m_t), take_t = exp(i_t - m_t); a normaliser n_t = keep_t n_(t-1) + take_t k_t
@@ -41,10 +41,23 @@ struct MemArgs {
   float* out;            // [tokens, out_rs]: head h at columns h * vdim
   int64_t out_rs;
   int H, dim, vdim, per_head, silu;
-  float q_scale, cap;
+  float q_scale, k_scale, cap;
+  const float* rot;      // [tokens, rot_dims]: cosines then sines of the tokens' angles, read when rot_dims > 0
+  int rot_dims;          // the first rot_dims numbers of q and k turn, number i with i + rot_dims / 2
 };
 
 __device__ __forceinline__ float maybe_silu(float z, int on) { return on ? silu_f32(z) : z; }
+
+// number i of the q or k vector at src (activated), turned by the token's angles
+__device__ __forceinline__ float turned(const MemArgs& p, const float* src, int i, const float* rot_row) {
+  const float x = maybe_silu(src[i], p.silu);
+  if (i >= p.rot_dims) return x;
+  const int half = p.rot_dims >> 1;
+  const bool first = i < half;
+  const int f = first ? i : i - half;
+  const float other = maybe_silu(src[first ? i + half : f], p.silu), c = rot_row[f], s = rot_row[half + f];
+  return first ? x * c - other * s : x * c + other * s;
+}
 
 constexpr int MEM_SLICE = 64;      // state columns that share one copy of n | m
 
@@ -94,13 +107,13 @@ __global__ __launch_bounds__(256) void matrix_memory_kernel(MemArgs p) {
     for (int base = tid * 4; base < nt * DMAX; base += nthr * 4) {
       const int j = base / DMAX, i = base % DMAX;          // DMAX is a multiple of 4: the four share a token
       float k4[4], q4[4];
-      const float* row = p.proj + (int64_t)(c0 + j) * p.proj_rs;
+      const float* row = p.proj + (int64_t)(c0 + j) * p.proj_rs + h * p.dim;
+      const float* rot_row = p.rot + (int64_t)(c0 + j) * p.rot_dims;
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const bool in = i + e < p.dim;
-        const int ch = h * p.dim + (in ? i + e : 0);
-        k4[e] = in ? maybe_silu(row[p.k_off + ch], p.silu) : 0.0f;
-        q4[e] = in ? maybe_silu(row[p.q_off + ch], p.silu) * p.q_scale : 0.0f;
+        k4[e] = in ? turned(p, row + p.k_off, i + e, rot_row) * p.k_scale : 0.0f;
+        q4[e] = in ? turned(p, row + p.q_off, i + e, rot_row) * p.q_scale : 0.0f;
       }
       *reinterpret_cast<float4*>(sk + base) = make_float4(k4[0], k4[1], k4[2], k4[3]);
       *reinterpret_cast<float4*>(sq + base) = make_float4(q4[0], q4[1], q4[2], q4[3]);
@@ -222,8 +235,9 @@ __global__ __launch_bounds__(256) void matrix_memory_generic_kernel(MemArgs p) {
   for (int t = t0; t < t1; ++t) {
     const float* row = p.proj + (int64_t)t * p.proj_rs;
     for (int i = tid; i < p.dim; i += nthr) {
-      sk[i] = maybe_silu(row[p.k_off + h * p.dim + i], p.silu);
-      sq[i] = maybe_silu(row[p.q_off + h * p.dim + i], p.silu) * p.q_scale;
+      const float* rot_row = p.rot + (int64_t)t * p.rot_dims;
+      sk[i] = turned(p, row + p.k_off + h * p.dim, i, rot_row) * p.k_scale;
+      sq[i] = turned(p, row + p.q_off + h * p.dim, i, rot_row) * p.q_scale;
     }
     if (tid == 0) {
       if constexpr (MODE == MEM_EXPGATE) {
@@ -310,13 +324,15 @@ extern "C" int64_t nv_matrix_memory_state_size(int mode, int dim, int vdim) {
 extern "C" int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int i_off,
                                 int f_off, const void* bias, const float* decay, float* state, const int32_t* cu_q,
                                 const int32_t* past_lens, const int32_t* state_slots, float* out, int64_t out_row_stride,
-                                int num_seqs, int heads, int dim, int vdim, int mode, int silu, float q_scale, float cap,
-                                int dtype, nv_stream_t stream) {
+                                int num_seqs, int heads, int dim, int vdim, int mode, int silu, float q_scale,
+                                float k_scale, const float* rot, int rot_dims, float cap, int dtype, nv_stream_t stream) {
   NV_CHECK_ARG(proj && state && cu_q && past_lens && state_slots && out, "nv_matrix_memory: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_matrix_memory: bad dtype %d", dtype);
   NV_CHECK_ARG(mode == MEM_CONST || mode == MEM_EXPGATE, "nv_matrix_memory: bad mode %d", mode);
   NV_CHECK_ARG(mode != MEM_CONST || decay, "nv_matrix_memory: constant decays are missing");
   NV_CHECK_ARG(mode != MEM_EXPGATE || cap > 0.0f, "nv_matrix_memory: the gate cap must be positive");
+  NV_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || rot),
+               "nv_matrix_memory: a rotation over %d of %d numbers needs its cosines and sines", rot_dims, dim);
   NV_CHECK_ARG(heads > 0 && heads <= 65535 && dim > 0 && vdim > 0 && num_seqs >= 0 && num_seqs <= 65535,
                "nv_matrix_memory: bad shape heads=%d dim=%d vdim=%d seqs=%d", heads, dim, vdim, num_seqs);
   if (num_seqs == 0) return NV_OK;
@@ -339,7 +355,8 @@ extern "C" int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int 
   }
   const int threads = vdp * cs;
   MemArgs p{proj, proj_row_stride, q_off, k_off, v_off, i_off, f_off, bias, decay, state, cu_q, past_lens, state_slots,
-            out, out_row_stride, heads, dim, vdim, (int)nv_matrix_memory_state_size(mode, dim, vdim), silu, q_scale, cap};
+            out, out_row_stride, heads, dim, vdim, (int)nv_matrix_memory_state_size(mode, dim, vdim), silu, q_scale, k_scale, cap,
+            rot, rot_dims};
   if (dmax > 256 || slices > 65535 || getenv("NV_MATRIX_MEMORY_GENERIC") != nullptr) {
     const size_t glds = ((size_t)2 * dim + 4 + 32) * sizeof(float);
     NV_CHECK_ARG(glds <= 64 * 1024, "nv_matrix_memory: keys of %d numbers exceed the LDS", dim);

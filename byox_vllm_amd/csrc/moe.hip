@@ -1,62 +1,133 @@
 // Mixture-of-experts bookkeeping around the grouped products of nv_linear:
 //   nv_moe_route   : per token the `top` largest router logits (fp32) and the softmax over just those (mode 0), or
 //                    the softmax over all experts, the chosen scores divided by (their sum + 1e-20) (mode 1), or
-//                    the sigmoid of each chosen logit as it is (mode 2)
+//                    the sigmoid of each chosen logit as it is (mode 2), or the softmax over all experts as it is (mode 3)
 //   nv_moe_sort    : (token, choice) pairs ordered by expert -> group offsets, the token behind every sorted row and
 //                    the sorted row of every pair
 //   nv_moe_plan    : both, in one launch for short steps, with the weight of every sorted row and a shared expert that
-//                    every token has as its last choice
+//                    every token has as its last choice.  Options of the choice (modes 1 - 3): a correction added to the
+//                    scores where they are compared, only the best groups of neighbouring experts to choose from, a
+//                    factor on the weights, and router outputs behind the experts whose "expert" is the identity: they
+//                    take part in everything but own no rows, a token's weights of them are summed instead
 //   nv_moe_combine : weighted sum of a token's expert rows (+ a sigmoid-gated shared expert)
 // The sum over a token's experts runs in the order of its choices, so it does not depend on what else is in the batch.
 #include "anyt.h"
 
 namespace {
 
-// One wavefront routes one token.  Choices come out in descending order, ties go to the lower index: the next choice is
-// the best among what comes after the previous one in that order, so nothing has to be marked as taken.
-__device__ __forceinline__ void route_token(const float* __restrict__ row, int E, int top, int mode, int32_t* ti, float* tw,
-                                            int lane) {
-  constexpr int NONE = 0x7fffffff;
+constexpr int ROUTE_NONE = 0x7fffffff;
+
+// How a token's experts are chosen and weighed.  ``n`` counts the router's outputs, identity experts included.
+struct RouteArgs {
+  int n, top, mode;
+  const float* correction;   // [n] added to the scores where they are compared (not to the weights), or null
+  int groups, keep;          // > 0: n / groups neighbours form a group; only the `keep` groups with the best member count
+  float scale;               // factor on the weights
+  // the choice compares scores (kept in LDS, n numbers per wavefront) and not plain logits
+  __host__ __device__ bool scored() const { return correction != nullptr || groups > 0; }
+};
+
+// The best of v[0 .. n) that comes after (pv, pe) in descending order, ties to the lower index: taking one after the
+// other this way, nothing has to be marked as taken.  Every lane of the wavefront gets the result.
+__device__ __forceinline__ void next_best(const float* v, int n, int lane, float pv, int pe, float& bv, int& be) {
+  bv = -INFINITY;
+  be = ROUTE_NONE;
+  for (int e = lane; e < n; e += 64) {
+    const float x = v[e];
+    if ((x < pv || (x == pv && e > pe)) && (be == ROUTE_NONE || x > bv)) {
+      bv = x;
+      be = e;
+    }
+  }
+#pragma unroll
+  for (int o = 1; o < 64; o <<= 1) {
+    const float v2 = __shfl_xor(bv, o, 64);
+    const int e2 = __shfl_xor(be, o, 64);
+    if (e2 != ROUTE_NONE && (be == ROUTE_NONE || v2 > bv || (v2 == bv && e2 < be))) {
+      bv = v2;
+      be = e2;
+    }
+  }
+}
+
+// LDS written by one lane and read by another of the same wavefront
+__device__ __forceinline__ void wave_lds_fence() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// One wavefront routes one token.  Choices come out in descending order.  ``lds``: n + groups numbers of this wavefront,
+// used when p.scored().
+__device__ __forceinline__ void route_token(const float* __restrict__ row, const RouteArgs& p, int32_t* ti, float* tw,
+                                            float* lds, int lane) {
+  const int n = p.n, top = p.top, mode = p.mode;
+  float all = 0.0f, m = 0.0f;
+  if (mode == 1 || mode == 3) {
+    m = -INFINITY;
+    for (int e = lane; e < n; e += 64) m = fmaxf(m, row[e]);
+    m = wave_max(m);
+    for (int e = lane; e < n; e += 64) all += expf(row[e] - m);
+    all = wave_sum(all);
+  }
+  const float* compare = row;
+  const bool scored = p.scored();
+  if (scored) {
+    float* best = lds + n;           // [groups] best member of each group
+    for (int e = lane; e < n; e += 64) {
+      const float s = mode == 2 ? sigmoid_f32(row[e]) : expf(row[e] - m) / all;
+      lds[e] = s + (p.correction ? p.correction[e] : 0.0f);
+    }
+    wave_lds_fence();
+    if (p.groups > 0 && p.keep < p.groups) {
+      const int size = n / p.groups;
+      for (int g = lane; g < p.groups; g += 64) {
+        float b = -INFINITY;
+        for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, lds[e]);
+        best[g] = b;
+      }
+      wave_lds_fence();
+      float pv = INFINITY;
+      int pe = -1;
+      for (int j = 0; j < p.keep; ++j) {
+        float bv;
+        int be;
+        next_best(best, p.groups, lane, pv, pe, bv, be);
+        if (be == ROUTE_NONE) break;
+        pv = bv;
+        pe = be;
+      }
+      // (pv, pe) is the last group kept
+      for (int e = lane; e < n; e += 64) {
+        const int g = e / size;
+        if (best[g] < pv || (best[g] == pv && g > pe)) lds[e] = -INFINITY;
+      }
+      wave_lds_fence();
+    }
+    compare = lds;
+  }
   float pv = INFINITY;
   int pe = -1;
   for (int j = 0; j < top; ++j) {
-    float bv = -INFINITY;
-    int be = NONE;
-    for (int e = lane; e < E; e += 64) {
-      const float v = row[e];
-      if ((v < pv || (v == pv && e > pe)) && (be == NONE || v > bv)) {
-        bv = v;
-        be = e;
-      }
-    }
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const float v2 = __shfl_xor(bv, o, 64);
-      const int e2 = __shfl_xor(be, o, 64);
-      if (e2 != NONE && (be == NONE || v2 > bv || (v2 == bv && e2 < be))) {
-        bv = v2;
-        be = e2;
-      }
-    }
-    if (be == NONE) be = j;          // only logits that are no numbers: any expert within range
+    float bv;
+    int be;
+    next_best(compare, n, lane, pv, pe, bv, be);
+    if (be == ROUTE_NONE) be = j;    // only logits that are no numbers: any expert within range
     if (lane == 0) {
       ti[j] = be;
-      tw[j] = bv;
+      tw[j] = scored ? row[be] : bv;
     }
     pv = bv;
     pe = be;
   }
-  float all = 0.0f, m = 0.0f;
-  if (mode == 1) {
-    m = -INFINITY;
-    for (int e = lane; e < E; e += 64) m = fmaxf(m, row[e]);
-    m = wave_max(m);
-    for (int e = lane; e < E; e += 64) all += expf(row[e] - m);
-    all = wave_sum(all);
-  }
+  if (scored) wave_lds_fence();      // the next token's scores take this one's place
   if (lane != 0) return;
   if (mode == 2) {                   // the sigmoid of each chosen logit, as it is
-    for (int j = 0; j < top; ++j) tw[j] = sigmoid_f32(tw[j]);
+    for (int j = 0; j < top; ++j) tw[j] = sigmoid_f32(tw[j]) * p.scale;
+    return;
+  }
+  if (mode == 3) {                   // scores of the softmax over every expert, as they are
+    for (int j = 0; j < top; ++j) tw[j] = expf(tw[j] - m) / all * p.scale;
     return;
   }
   float sum = 0.0f;
@@ -65,7 +136,7 @@ __device__ __forceinline__ void route_token(const float* __restrict__ row, int E
       tw[j] = expf(tw[j] - m) / all;
       sum += tw[j];
     }
-    for (int j = 0; j < top; ++j) tw[j] /= sum + 1e-20f;
+    for (int j = 0; j < top; ++j) tw[j] = tw[j] / (sum + 1e-20f) * p.scale;
     return;
   }
   m = tw[0];
@@ -73,15 +144,17 @@ __device__ __forceinline__ void route_token(const float* __restrict__ row, int E
     tw[j] = expf(tw[j] - m);
     sum += tw[j];
   }
-  for (int j = 0; j < top; ++j) tw[j] /= sum;
+  for (int j = 0; j < top; ++j) tw[j] = tw[j] / sum * p.scale;
 }
 
-__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t rs, int E, int top,
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t rs,
                                                         int32_t* __restrict__ idx, float* __restrict__ wt, int64_t T_,
-                                                        int mode) {
-  const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+                                                        RouteArgs p) {
+  extern __shared__ float scores[];                                  // 4 x (n + groups) when the choice compares scores
+  const int wv = threadIdx.x >> 6;
+  const int64_t t = (int64_t)blockIdx.x * 4 + wv;
   if (t >= T_) return;
-  route_token(logits + t * rs, E, top, mode, idx + t * top, wt + t * top, threadIdx.x & 63);
+  route_token(logits + t * rs, p, idx + t * p.top, wt + t * p.top, scores + wv * (p.n + p.groups), threadIdx.x & 63);
 }
 
 struct SortArgs {
@@ -89,6 +162,7 @@ struct SortArgs {
   const float* wt;           // [tokens, top]
   int64_t tokens;
   int E, top, shared;        // shared 1: every token also has choice `top`, expert E with weight 1
+  float* self_weight;        // [tokens] sum of the weights of choices >= E (identity experts: no rows, slot -1), or null
   int32_t* offsets;          // [E + shared + 1]
   int32_t* sorted_token;     // [tokens * (top + shared)]
   float* sorted_weight;      // the same, or null
@@ -124,15 +198,28 @@ __device__ __forceinline__ void counts_to_starts(int32_t* cnt, const SortArgs& p
 __device__ __forceinline__ void scatter_pairs(int32_t* cnt, const int32_t* idx, const SortArgs& p) {
   const int64_t pairs = p.tokens * p.top;
   const int C = p.top + p.shared;
+  if (p.self_weight) {
+    for (int64_t t = threadIdx.x; t < p.tokens; t += blockDim.x) {
+      float w = 0.0f;
+      for (int j = 0; j < p.top; ++j)
+        if (idx[t * p.top + j] >= p.E) w += p.wt[t * p.top + j];
+      p.self_weight[t] = w;
+    }
+  }
   for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x) {
+    if (idx[i] >= p.E) {
+      p.slot_of[i / p.top * C + i % p.top] = -1;
+      continue;
+    }
     const int slot = atomicAdd(&cnt[idx[i]], 1);
     p.sorted_token[slot] = (int32_t)(i / p.top);
     if (p.sorted_weight) p.sorted_weight[slot] = p.wt[i];
     p.slot_of[i / p.top * C + i % p.top] = slot;
   }
   if (!p.shared) return;
+  const int64_t routed = p.offsets[p.E];             // written before the barrier ahead of this call
   for (int64_t t = threadIdx.x; t < p.tokens; t += blockDim.x) {
-    const int64_t slot = pairs + t;
+    const int64_t slot = routed + t;
     p.sorted_token[slot] = (int32_t)t;
     if (p.sorted_weight) p.sorted_weight[slot] = 1.0f;
     p.slot_of[t * C + p.top] = (int32_t)slot;
@@ -144,7 +231,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(SortArgs p) {
   const int64_t pairs = p.tokens * p.top;
   for (int e = threadIdx.x; e < p.E; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
-  for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x) atomicAdd(&cnt[p.idx[i]], 1);
+  for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x)
+    if (p.idx[i] < p.E) atomicAdd(&cnt[p.idx[i]], 1);
   __syncthreads();
   counts_to_starts(cnt, p);
   __syncthreads();
@@ -152,18 +240,19 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(SortArgs p) {
 }
 
 // routing and ordering of a short step in one launch: sixteen wavefronts route a token each, then sort together
-__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ logits, int64_t rs, int mode, int32_t* idx_out,
-                                                        float* wt_out, SortArgs p) {
-  extern __shared__ int32_t cnt[];                                   // [E] | choices [tokens * top] | their weights
+__global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ logits, int64_t rs, int32_t* idx_out,
+                                                        float* wt_out, SortArgs p, RouteArgs r) {
+  extern __shared__ int32_t cnt[];                  // [E] | choices [tokens * top] | their weights | 16 x (n + groups) scores
   int32_t* choice = cnt + p.E;
   const int64_t pairs = p.tokens * p.top;
   float* weight = reinterpret_cast<float*>(choice + pairs);
+  float* scores = weight + pairs + (threadIdx.x >> 6) * (r.n + r.groups);
   for (int e = threadIdx.x; e < p.E; e += blockDim.x) cnt[e] = 0;
   for (int64_t t = threadIdx.x >> 6; t < p.tokens; t += blockDim.x >> 6)
-    route_token(logits + t * rs, p.E, p.top, mode, choice + t * p.top, weight + t * p.top, threadIdx.x & 63);
+    route_token(logits + t * rs, r, choice + t * p.top, weight + t * p.top, scores, threadIdx.x & 63);
   __syncthreads();
   for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x) {
-    atomicAdd(&cnt[choice[i]], 1);
+    if (choice[i] < p.E) atomicAdd(&cnt[choice[i]], 1);
     idx_out[i] = choice[i];
     wt_out[i] = weight[i];
   }
@@ -182,7 +271,10 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
   const float gate = !shared ? 0.0f : sg ? sigmoid_f32(sg[t * sg_rs]) : 1.0f;   // no gate logits: a plain addend
   for (int c = threadIdx.x; c < width; c += blockDim.x) {
     float a = 0.0f;
-    for (int j = 0; j < top; ++j) a += wt[t * top + j] * y[(int64_t)slot_of[t * top + j] * width + c];
+    for (int j = 0; j < top; ++j) {
+      const int slot = slot_of[t * top + j];
+      if (slot >= 0) a += wt[t * top + j] * y[(int64_t)slot * width + c];
+    }
     if (shared) a += gate * shared[t * width + c];
     out[t * width + c] = a;
   }
@@ -193,12 +285,12 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
 extern "C" int nv_moe_route(const float* logits, int64_t row_stride, int32_t* idx, float* weights, int64_t tokens,
                             int experts, int top, int mode, nv_stream_t stream) {
   NV_CHECK_ARG(logits && idx && weights, "nv_moe_route: null pointer");
-  NV_CHECK_ARG(mode >= 0 && mode <= 2, "nv_moe_route: bad mode %d", mode);
+  NV_CHECK_ARG(mode >= 0 && mode <= 3, "nv_moe_route: bad mode %d", mode);
   NV_CHECK_ARG(tokens >= 0 && experts > 0 && top > 0 && top <= experts, "nv_moe_route: bad shape experts=%d top=%d",
                experts, top);
   if (tokens == 0) return NV_OK;
   moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 0, (hipStream_t)stream>>>(
-      logits, row_stride, experts, top, idx, weights, tokens, mode);
+      logits, row_stride, idx, weights, tokens, RouteArgs{experts, top, mode, nullptr, 0, 0, 1.0f});
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
@@ -207,30 +299,39 @@ extern "C" int nv_moe_sort(const int32_t* idx, int64_t tokens, int experts, int 
                            int32_t* sorted_token, int32_t* slot_of, nv_stream_t stream) {
   NV_CHECK_ARG(idx && offsets && sorted_token && slot_of, "nv_moe_sort: null pointer");
   NV_CHECK_ARG(tokens >= 0 && experts > 0 && experts <= 8192 && top > 0, "nv_moe_sort: bad shape");
-  SortArgs p{idx, nullptr, tokens, experts, top, 0, offsets, sorted_token, nullptr, slot_of};
+  SortArgs p{idx, nullptr, tokens, experts, top, 0, nullptr, offsets, sorted_token, nullptr, slot_of};
   moe_sort_kernel<<<dim3(1), dim3(1024), (size_t)experts * sizeof(int32_t), (hipStream_t)stream>>>(p);
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
 
 extern "C" int nv_moe_plan(const float* logits, int64_t row_stride, int64_t tokens, int experts, int top, int mode, int shared,
-                           int32_t* idx, float* weights, int32_t* offsets, int32_t* sorted_token, float* sorted_weight,
-                           int32_t* slot_of, nv_stream_t stream) {
+                           int identity, const float* correction, int groups, int keep_groups, float scale, int32_t* idx,
+                           float* weights, int32_t* offsets, int32_t* sorted_token, float* sorted_weight, int32_t* slot_of,
+                           float* self_weight, nv_stream_t stream) {
   NV_CHECK_ARG(logits && idx && weights && offsets && sorted_token && slot_of, "nv_moe_plan: null pointer");
-  NV_CHECK_ARG(mode >= 0 && mode <= 2 && (shared == 0 || shared == 1), "nv_moe_plan: bad mode %d / %d", mode, shared);
-  NV_CHECK_ARG(tokens >= 0 && tokens * (top + 1) < (1ll << 31) && experts > 0 && experts <= 8192 && top > 0 && top <= experts,
-               "nv_moe_plan: bad shape experts=%d top=%d", experts, top);
+  NV_CHECK_ARG(mode >= 0 && mode <= 3 && (shared == 0 || shared == 1), "nv_moe_plan: bad mode %d / %d", mode, shared);
+  NV_CHECK_ARG(tokens >= 0 && tokens * (top + 1) < (1ll << 31) && experts > 0 && identity >= 0 && experts + identity <= 8192 &&
+                   top > 0 && top <= experts + identity,
+               "nv_moe_plan: bad shape experts=%d identity=%d top=%d", experts, identity, top);
+  NV_CHECK_ARG((identity == 0) == (self_weight == nullptr), "nv_moe_plan: identity experts need self_weight");
+  const RouteArgs r{experts + identity, top, mode, correction, groups, keep_groups, scale};
+  NV_CHECK_ARG(!r.scored() || mode != 0, "nv_moe_plan: mode 0 has no scores to correct or group");
+  NV_CHECK_ARG(groups >= 0 && (groups == 0 || (r.n % groups == 0 && keep_groups > 0 && keep_groups <= groups &&
+                                               keep_groups * (r.n / groups) >= top)),
+               "nv_moe_plan: bad groups %d / %d", groups, keep_groups);
   if (tokens == 0) return NV_OK;
   hipStream_t s = (hipStream_t)stream;
-  SortArgs p{idx, weights, tokens, experts, top, shared, offsets, sorted_token, sorted_weight, slot_of};
-  if (tokens <= 64 && tokens * top <= 2048) {
-    const size_t lds = (experts + 2 * tokens * top) * sizeof(int32_t);
-    moe_plan_kernel<<<dim3(1), dim3(1024), lds, s>>>(logits, row_stride, mode, idx, weights, p);
+  SortArgs p{idx, weights, tokens, experts, top, shared, self_weight, offsets, sorted_token, sorted_weight, slot_of};
+  const size_t scores = r.scored() ? (size_t)(r.n + groups) * sizeof(float) : 0;      // per wavefront
+  const size_t plan_lds = (experts + 2 * tokens * top) * sizeof(int32_t) + 16 * scores;
+  if (tokens <= 64 && tokens * top <= 2048 && plan_lds <= 64 * 1024) {
+    moe_plan_kernel<<<dim3(1), dim3(1024), plan_lds, s>>>(logits, row_stride, idx, weights, p, r);
     NV_CHECK_LAUNCH();
     return NV_OK;
   }
-  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 0, s>>>(logits, row_stride, experts, top, idx, weights,
-                                                                            tokens, mode);
+  NV_CHECK_ARG(4 * scores <= 64 * 1024, "nv_moe_plan: the scores of %d outputs exceed the LDS", r.n);
+  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 4 * scores, s>>>(logits, row_stride, idx, weights, tokens, r);
   NV_CHECK_LAUNCH();
   moe_sort_kernel<<<dim3(1), dim3(1024), (size_t)experts * sizeof(int32_t), s>>>(p);
   NV_CHECK_LAUNCH();

@@ -16,6 +16,21 @@ __global__ __launch_bounds__(256) void embed_scale_kernel(const int64_t* __restr
   for (int i = threadIdx.x; i < width; i += blockDim.x) out[t * width + i] = ld_f32<T>(row + i) * scale;
 }
 
+// out[t] = cosines then sines of position[t] * inv_freq[i], i < half.  The angle is formed and reduced in double: a float
+// angle of a position in the thousands is already off by 1e-4.
+__global__ __launch_bounds__(256) void rotation_table_kernel(const int64_t* __restrict__ positions,
+                                                             const double* __restrict__ inv_freq, float* __restrict__ out,
+                                                             int64_t total, int half) {
+  const int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total) return;
+  const int64_t t = i / half;
+  const int f = (int)(i % half);
+  double s, c;
+  sincos((double)positions[t] * inv_freq[f], &s, &c);
+  out[t * 2 * half + f] = (float)c;
+  out[t * 2 * half + half + f] = (float)s;
+}
+
 // v = x[r] + delta[r] (when delta is given; written back to x unless rows are gathered), out[i] = tanh(alpha * v) * w + b
 // with r = rows_idx ? rows_idx[i] : i
 template <typename T>
@@ -196,6 +211,8 @@ struct SandwichArgs {
   const float* shared;       // [.., n] more rows to add, times sigmoid(shared_gate), or null
   const float* shared_gate;
   int64_t shared_gate_rs;
+  const void* self;          // [.., n] rows in the storage type to add, times self_weight (identity experts), or null
+  const float* self_weight;  // [..]
   int n;
   float eps;
 };
@@ -212,6 +229,7 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(SandwichArgs p) {
   const int n = p.n, tid = threadIdx.x;
   float* xr = p.x + t * n;
   const float gate = p.shared ? sigmoid_f32(p.shared_gate[t * p.shared_gate_rs]) : 0.0f;
+  const float self_w = p.self ? p.self_weight[t] : 0.0f;
   const float last = p.slot_of && p.last_gate ? sigmoid_f32(p.last_gate[t * p.last_gate_rs]) : 1.0f;
   f32x4 v[STEPS];
   auto load4 = [](const float* q, int c) { return *reinterpret_cast<const f32x4*>(q + c); };
@@ -227,8 +245,10 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(SandwichArgs p) {
       for (int k = 0; k < STEPS; ++k) v[k] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
       if (p.slot_of) {
         for (int q = 0; q < p.choices; ++q) {
+          const int slot = p.slot_of[t * p.choices + q];
+          if (slot < 0) continue;              // an identity expert: no row
           const float f = factor(q);
-          const float* yr = p.y + (int64_t)p.slot_of[t * p.choices + q] * p.y_rs;
+          const float* yr = p.y + (int64_t)slot * p.y_rs;
 #pragma unroll
           for (int k = 0; k < STEPS; ++k) {
             const int c = (tid + k * 256) * 4;
@@ -255,6 +275,11 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(SandwichArgs p) {
 #pragma unroll
           for (int e = 0; e < 4; ++e) v[k][e] += gate * a[e];
         }
+        if (p.self) {
+          const f32x4 a = widen4(reinterpret_cast<const T*>(p.self) + t * n, c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) v[k][e] += self_w * a[e];
+        }
         if (p.y_bias) {
           const f32x4 b = widen4(p.y_bias, c);
 #pragma unroll
@@ -267,11 +292,15 @@ __global__ __launch_bounds__(256) void sandwich_norm_kernel(SandwichArgs p) {
       for (int c = tid; c < n; c += 256) {
         float a = 0.0f;
         if (p.slot_of) {
-          for (int q = 0; q < p.choices; ++q) a += factor(q) * p.y[(int64_t)p.slot_of[t * p.choices + q] * p.y_rs + c];
+          for (int q = 0; q < p.choices; ++q) {
+            const int slot = p.slot_of[t * p.choices + q];
+            if (slot >= 0) a += factor(q) * p.y[(int64_t)slot * p.y_rs + c];
+          }
         } else {
           a = p.y[t * p.y_rs + c];
         }
         if (p.shared) a += gate * p.shared[t * n + c];
+        if (p.self) a += self_w * ld_f32<T>(reinterpret_cast<const T*>(p.self) + t * n + c);
         if (p.y_bias) a += ld_f32<T>(reinterpret_cast<const T*>(p.y_bias) + c);
         row_lds[c] = a;
         ss += a * a;
@@ -465,8 +494,10 @@ extern "C" int nv_sandwich_norm(float* x, const float* y, int64_t y_row_stride, 
                                 const void* w_pre, void* out, int64_t out_row_stride, const int32_t* rows_idx,
                                 const int32_t* slot_of, int choices, const float* weights, const float* last_gate,
                                 int64_t last_gate_stride, const float* shared, const float* shared_gate,
-                                int64_t shared_gate_stride, int64_t rows, int n, float eps, int dtype, nv_stream_t stream) {
-  NV_CHECK_ARG(x && (y || !(y_bias || w_post || slot_of || shared)), "nv_sandwich_norm: null pointer");
+                                int64_t shared_gate_stride, const void* self, const float* self_weight, int64_t rows, int n,
+                                float eps, int dtype, nv_stream_t stream) {
+  NV_CHECK_ARG(x && (y || !(y_bias || w_post || slot_of || shared || self)), "nv_sandwich_norm: null pointer");
+  NV_CHECK_ARG(!self || self_weight, "nv_sandwich_norm: self rows need their weights");
   NV_CHECK_ARG((w_pre == nullptr) == (out == nullptr) && (w_pre || (y && !rows_idx)), "nv_sandwich_norm: nothing to do");
   NV_CHECK_ARG(!slot_of || choices > 0, "nv_sandwich_norm: bad choices %d", choices);
   NV_CHECK_ARG(!shared || shared_gate, "nv_sandwich_norm: shared rows need their gate");
@@ -474,10 +505,10 @@ extern "C" int nv_sandwich_norm(float* x, const float* y, int64_t y_row_stride, 
   NV_CHECK_ARG(rows >= 0 && rows < (1ll << 31) && n > 0 && n <= 16000, "nv_sandwich_norm: bad shape, rows of %d numbers", n);
   if (rows == 0) return NV_OK;
   SandwichArgs p{x, y, y_row_stride, y_bias, w_post, w_pre, out, out_row_stride, rows_idx, slot_of, choices, weights,
-                 last_gate, last_gate_stride, shared, shared_gate, shared_gate_stride, n, eps};
+                 last_gate, last_gate_stride, shared, shared_gate, shared_gate_stride, self, self_weight, n, eps};
   auto al16 = [](const void* q) { return ((uintptr_t)q & 15) == 0; };
   const bool vec = n % 4 == 0 && n <= 4096 && al16(x) && al16(y) && al16(y_bias) && al16(w_post) && al16(w_pre) && al16(out) &&
-                   al16(shared) && (!y || y_row_stride % 4 == 0) && out_row_stride % 4 == 0;
+                   al16(shared) && al16(self) && (!y || y_row_stride % 4 == 0) && out_row_stride % 4 == 0;
   hipStream_t s = (hipStream_t)stream;
 #define NV_SANDWICH(NVAL, LDS) \
   NV_DISPATCH_T(dtype, sandwich_norm_kernel<T, NVAL><<<dim3((unsigned)rows), dim3(256), LDS, s>>>(p))
@@ -554,6 +585,18 @@ extern "C" int nv_embed_scale(const int64_t* ids, const void* table, float* out,
   if (tokens == 0) return NV_OK;
   NV_DISPATCH_T(dtype, embed_scale_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(
                            ids, (const T*)table, out, width, vocab, scale));
+  NV_CHECK_LAUNCH();
+  return NV_OK;
+}
+
+extern "C" int nv_rotation_table(const int64_t* positions, const double* inv_freq, float* out, int64_t tokens, int half,
+                                 nv_stream_t stream) {
+  NV_CHECK_ARG(positions && inv_freq && out, "nv_rotation_table: null pointer");
+  NV_CHECK_ARG(tokens >= 0 && half > 0 && tokens * half < (1ll << 38), "nv_rotation_table: bad shape");
+  if (tokens == 0) return NV_OK;
+  const int64_t total = tokens * half;
+  rotation_table_kernel<<<dim3((unsigned)((total + 255) / 256)), dim3(256), 0, (hipStream_t)stream>>>(positions, inv_freq, out,
+                                                                                                     total, half);
   NV_CHECK_LAUNCH();
   return NV_OK;
 }

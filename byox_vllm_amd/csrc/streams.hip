@@ -144,7 +144,8 @@ template <typename T>
 __global__ __launch_bounds__(256) void group_rmsnorm_f32_kernel(const float* __restrict__ x, int64_t x_rs,
                                                                 const T* __restrict__ w, T* __restrict__ out,
                                                                 int64_t out_rs, int groups, int n, float eps,
-                                                                const float* __restrict__ gate, int64_t gate_rs) {
+                                                                const float* __restrict__ gate, int64_t gate_rs,
+                                                                int gate_silu) {
   __shared__ float red[32];
   const int64_t t = blockIdx.x / groups;
   const int g = blockIdx.x % groups;
@@ -154,8 +155,11 @@ __global__ __launch_bounds__(256) void group_rmsnorm_f32_kernel(const float* __r
   ss = block_sum(ss, red);
   const float inv = 1.0f / sqrtf(ss / (float)n + eps);
   for (int j = threadIdx.x; j < n; j += blockDim.x) {
-    float v = xr[j] * inv * ld_f32<T>(w + (int64_t)g * n + j);
-    if (gate) v *= sigmoid_f32(gate[t * gate_rs + (int64_t)g * n + j]);
+    float v = xr[j] * inv * (w ? ld_f32<T>(w + (int64_t)g * n + j) : 1.0f);
+    if (gate) {
+      const float z = gate[t * gate_rs + (int64_t)g * n + j];
+      v *= gate_silu ? silu_f32(z) : sigmoid_f32(z);
+    }
     st_f32<T>(out + t * out_rs + (int64_t)g * n + j, v);
   }
 }
@@ -166,7 +170,7 @@ __global__ __launch_bounds__(256) void group_rmsnorm_f32_wave_kernel(const float
                                                                      const T* __restrict__ w, T* __restrict__ out,
                                                                      int64_t out_rs, int64_t parts, int groups, int n,
                                                                      float eps, const float* __restrict__ gate,
-                                                                     int64_t gate_rs) {
+                                                                     int64_t gate_rs, int gate_silu) {
   const int64_t part = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (part >= parts) return;
   const int lane = threadIdx.x & 63;
@@ -186,8 +190,11 @@ __global__ __launch_bounds__(256) void group_rmsnorm_f32_wave_kernel(const float
   for (int i = 0; i < 4; ++i) {
     const int j = lane + 64 * i;
     if (j >= n) continue;
-    float y = v[i] * inv * ld_f32<T>(w + (int64_t)g * n + j);
-    if (gate) y *= sigmoid_f32(gate[t * gate_rs + (int64_t)g * n + j]);
+    float y = v[i] * inv * (w ? ld_f32<T>(w + (int64_t)g * n + j) : 1.0f);
+    if (gate) {
+      const float z = gate[t * gate_rs + (int64_t)g * n + j];
+      y *= gate_silu ? silu_f32(z) : sigmoid_f32(z);
+    }
     st_f32<T>(out + t * out_rs + (int64_t)g * n + j, y);
   }
 }
@@ -251,8 +258,8 @@ extern "C" int nv_token_shift(const float* h, const void* mu, float* state, cons
 
 extern "C" int nv_group_rmsnorm_f32(const float* x, int64_t x_row_stride, const void* w, void* out, int64_t out_row_stride,
                                     int64_t rows, int groups, int n, float eps, const float* gate,
-                                    int64_t gate_row_stride, int dtype, nv_stream_t stream) {
-  NV_CHECK_ARG(x && w && out, "nv_group_rmsnorm_f32: null pointer");
+                                    int64_t gate_row_stride, int gate_silu, int dtype, nv_stream_t stream) {
+  NV_CHECK_ARG(x && out, "nv_group_rmsnorm_f32: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_group_rmsnorm_f32: bad dtype %d", dtype);
   NV_CHECK_ARG(rows >= 0 && n > 0 && groups > 0 && rows * groups < (1ll << 31), "nv_group_rmsnorm_f32: bad shape");
   if (rows == 0) return NV_OK;
@@ -261,12 +268,13 @@ extern "C" int nv_group_rmsnorm_f32(const float* x, int64_t x_row_stride, const 
     NV_DISPATCH_T(dtype, group_rmsnorm_f32_wave_kernel<T><<<dim3((unsigned)((parts + 3) / 4)), dim3(256), 0,
                                                             (hipStream_t)stream>>>(
                              x, x_row_stride, (const T*)w, (T*)out, out_row_stride, parts, groups, n, eps, gate,
-                             gate_row_stride));
+                             gate_row_stride, gate_silu));
     NV_CHECK_LAUNCH();
     return NV_OK;
   }
   NV_DISPATCH_T(dtype, group_rmsnorm_f32_kernel<T><<<dim3((unsigned)(rows * groups)), dim3(256), 0, (hipStream_t)stream>>>(
-                           x, x_row_stride, (const T*)w, (T*)out, out_row_stride, groups, n, eps, gate, gate_row_stride));
+                           x, x_row_stride, (const T*)w, (T*)out, out_row_stride, groups, n, eps, gate, gate_row_stride,
+                           gate_silu));
   NV_CHECK_LAUNCH();
   return NV_OK;
 }

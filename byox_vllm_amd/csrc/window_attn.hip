@@ -21,6 +21,8 @@
 //
 // qk_pairs_store_kernel: the same where a number depends on itself and its neighbour only.
 //
+// qk_conv_store_kernel: the same behind a short causal convolution over time on every channel of q, k and v.
+//
 // window_attn_kernel: a workgroup owns TQ consecutive tokens of the packed batch and one key/value head, i.e. up to
 // TQ * (H / G) query rows that read the same keys; tokens of different requests inside the tile are served one request
 // after the other.  Keys go through LDS in tiles of TK rows; online softmax per row.
@@ -44,7 +46,8 @@ struct QkArgs {
   float* q_out;           // [tokens, H * d]
   int H, G, d, dv;
   float scale, eps;
-  int norm_whole;         // 1: one root mean square over all H * d query numbers (and over all G * d key numbers)
+  int norm_whole;         // 1: one root mean square over all H * d query numbers (and over all G * d key numbers);
+                          // 2: one per head, without weights
   const float* inv_freq;  // [rot_dims / 2] rotation frequencies, read when rot_dims > 0
   int rot_dims;           // the first rot_dims numbers of every head are rotated, dimension i with i + rot_dims / 2
   float mscale;           // multiplies cosine and sine
@@ -83,7 +86,7 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
     __syncthreads();
   }
   float inv_q = 1.0f, inv_k = 1.0f;
-  if (qn && p.norm_whole) {
+  if (qn && p.norm_whole == 1) {
     float sq = 0.0f, sk = 0.0f;
     for (int e = threadIdx.x; e < p.H * p.d; e += blockDim.x) {
       const float x = row[p.q_off + e] + (bias ? ld_f32<T>(bias + p.q_off + e) : 0.0f);
@@ -102,7 +105,7 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
     const int col = is_q ? p.q_off + hv * p.d : p.k_off + hv * p.d;
     const float* src = row + col;
     float inv = is_q ? inv_q : inv_k;
-    if (qn && !p.norm_whole) {
+    if (p.norm_whole == 2 || (qn && p.norm_whole == 0)) {
       float ss = 0.0f;
       for (int e = lane; e < p.d; e += 64) {
         const float x = src[e] + (bias ? ld_f32<T>(bias + col + e) : 0.0f);
@@ -112,7 +115,7 @@ __global__ __launch_bounds__(256) void qk_norm_store_kernel(QkArgs p) {
       inv = 1.0f / sqrtf(ss / (float)p.d + p.eps);
     }
     const T* nw_ = is_q ? qn : kn;
-    if (nw_ && p.norm_whole) nw_ += hv * p.d;
+    if (nw_ && p.norm_whole == 1) nw_ += hv * p.d;
     auto normed = [&](int e) {
       const float x = src[e] + (bias ? ld_f32<T>(bias + col + e) : 0.0f);
       return x * inv * (nw_ ? ld_f32<T>(nw_ + e) : 1.0f);
@@ -195,6 +198,120 @@ __global__ __launch_bounds__(256) void qk_pairs_store_kernel(QkArgs p) {
       *reinterpret_cast<f32x4*>(p.q_out + t * nq + rel) = x;
     } else if (crow) {
       *reinterpret_cast<P*>(crow + (is_v ? nk : 0) + rel) = Pack4<T>::narrow(x);
+    }
+  }
+}
+
+// A short causal convolution per channel of q | k | v, y_t = sum_j w[c][j] x_(t - taps + 1 + j) with zeros ahead of the
+// sequence, then (optionally) every query and key head divided by its root mean square, then query scale and page store.
+// The last taps - 1 inputs of a request are its state.
+struct QkConvArgs {
+  const float* proj;      // [tokens, proj_rs]: q | k | v at the column offsets
+  int64_t proj_rs;
+  int q_off, k_off, v_off;
+  const void* w;          // [H d + G d + G dv, taps] in the storage type
+  int taps;
+  float* state;           // [slots, taps - 1, H d + G d + G dv]
+  const int32_t* cu_q;    // [B + 1]
+  const int32_t* past;    // [B]
+  const int32_t* slots;   // [B]
+  const int32_t* seq_of;  // [tokens]
+  const int32_t* slot_mapping;   // [tokens] cache row or -1
+  void* cache;            // [rows, G (d + dv)]
+  float* q_out;           // [tokens, H d]
+  int64_t tokens;
+  int H, G, d, dv, norm;
+  float scale, eps;
+  int L, v_units;         // lanes that share a head (a power of two, 4 L >= d); units of 4 L value channels
+};
+
+constexpr int QC_MAX_TAPS = 8;
+
+// d % 4 == 0 and dv % 4 == 0.  A unit of L lanes owns a query head, a key head or a run of value channels, four channels
+// per lane, and walks TT consecutive tokens with the last taps rows of its channels in registers.  The tokens that reach
+// back over their portion's start (its first taps - 1) are all served by the workgroup of the portion's FIRST token, which
+// reads the slot there and at once writes its new contents: a channel's accesses to the slot come from one thread.
+template <typename T, int MAXT>
+__global__ __launch_bounds__(256) void qk_conv_store_kernel(QkConvArgs p, int TT) {
+  typedef typename Pack4<T>::type P;
+  const int L = p.L, unit = blockIdx.y * (256 / L) + threadIdx.x / L, e = (threadIdx.x % L) * 4;
+  const int taps = p.taps, keep = taps - 1;
+  const int nq = p.H * p.d, nk = p.G * p.d, nv = p.G * p.dv, C = nq + nk + nv;
+  const bool is_q = unit < p.H, is_v = unit >= p.H + p.G;
+  const int rel = is_v ? (unit - p.H - p.G) * 4 * L + e : (is_q ? unit : unit - p.H) * p.d + e;   // within q, k or v
+  const bool on = unit < p.H + p.G + p.v_units && (is_v ? rel < nv : e < p.d);
+  const int col = on ? (is_q ? p.q_off : is_v ? p.v_off : p.k_off) + rel : p.q_off;
+  const int ch = on ? (is_q ? 0 : is_v ? nq + nk : nq) + rel : 0;
+  const int64_t t_begin = (int64_t)blockIdx.x * TT, t_end = min(p.tokens, t_begin + TT);
+  f32x4 wt[MAXT], win[MAXT];        // inside the walk win[MAXT - 1 - m] is the row m tokens back
+  const T* w = reinterpret_cast<const T*>(p.w) + (int64_t)ch * taps;
+#pragma unroll
+  for (int m = 0; m < MAXT; ++m)    // wt[MAXT - 1 - m] multiplies the row m tokens back
+#pragma unroll
+    for (int i = 0; i < 4; ++i) wt[MAXT - 1 - m][i] = m < taps ? ld_f32<T>(w + i * taps + keep - m) : 0.0f;
+  auto row = [&](int64_t t) { return *reinterpret_cast<const f32x4*>(p.proj + max(t, (int64_t)0) * p.proj_rs + col); };
+  const f32x4 zero = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  // before the walk the window stands one token earlier
+  const int64_t t_first = p.cu_q[p.seq_of[t_begin]];
+#pragma unroll
+  for (int m = 1; m < MAXT; ++m) win[MAXT - m] = (m <= keep && t_begin - m >= t_first) ? row(t_begin - m) : zero;
+  win[0] = zero;
+  for (int64_t t = t_begin; t < p.tokens; ++t) {
+    const int b = p.seq_of[t];
+    const int64_t t0 = p.cu_q[b];
+    // past the tile: only the first tokens of a portion that began inside it
+    if (t >= t_end && !(t0 >= t_begin && t0 < t_end && t - t0 < keep)) break;
+    const f32x4 x = row(t);
+    if (t == t0 && keep > 0) {
+      float* slot = p.state + (int64_t)p.slots[b] * keep * C + ch;
+      const bool fresh = p.past[b] == 0;
+#pragma unroll
+      for (int m = 1; m < MAXT; ++m)       // slot row keep - m holds the input m tokens ahead of the portion
+        win[MAXT - m] = (m <= keep && on && !fresh) ? *reinterpret_cast<const f32x4*>(slot + (int64_t)(keep - m) * C) : zero;
+      if (on) {
+        const int n = p.cu_q[b + 1] - (int)t0;
+#pragma unroll
+        for (int m = 1; m < MAXT; ++m) {   // the new row keep - m: the input m - 1 tokens ahead of the portion's last one
+          if (m > keep) continue;
+          f32x4 v = zero;
+          if (n - m >= 0) {
+            v = row(t0 + n - m);
+          } else {
+#pragma unroll
+            for (int o = 1; o < MAXT; ++o)
+              if (o == m - n) v = win[MAXT - o];
+          }
+          *reinterpret_cast<f32x4*>(slot + (int64_t)(keep - m) * C) = v;
+        }
+      }
+    }
+#pragma unroll
+    for (int m = 0; m + 1 < MAXT; ++m) win[m] = win[m + 1];
+    win[MAXT - 1] = x;
+    if (t0 < t_begin && t - t0 < keep) continue;          // served by the workgroup of the portion's first token
+    f32x4 y = zero;
+#pragma unroll
+    for (int m = 0; m < MAXT; ++m) {
+      if (MAXT - 1 - m >= taps) continue;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) y[i] += wt[m][i] * win[m][i];
+    }
+    float f = 1.0f;
+    if (p.norm) {                                          // every lane of the wavefront takes part
+      float ss = on ? y[0] * y[0] + y[1] * y[1] + y[2] * y[2] + y[3] * y[3] : 0.0f;
+      for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
+      if (!is_v) f = 1.0f / sqrtf(ss / (float)p.d + p.eps);
+    }
+    if (!on) continue;
+    if (is_q) f *= p.scale;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) y[i] *= f;
+    if (is_q) {
+      *reinterpret_cast<f32x4*>(p.q_out + t * nq + rel) = y;
+    } else {
+      const int64_t slot = p.slot_mapping[t];
+      if (slot >= 0)
+        *reinterpret_cast<P*>(reinterpret_cast<T*>(p.cache) + slot * (nk + nv) + (is_v ? nk : 0) + rel) = Pack4<T>::narrow(y);
     }
   }
 }
@@ -928,7 +1045,8 @@ extern "C" int nv_qk_rotate_store(const float* proj, const void* bias, int64_t p
   NV_CHECK_ARG(!v_first || (vmix && vdim > 0), "nv_qk_store: blending values needs its weight");
   if (tokens == 0) return NV_OK;
   auto al = [](const void* q, size_t n) { return (uintptr_t)q % n == 0; };
-  const bool pairs = !q_norm && !temp && !bias && !v_first && temp_every == 0 && (rot_dims == 0 || (interleaved && rot_dims <= 256)) &&
+  NV_CHECK_ARG(norm_whole >= 0 && norm_whole <= 2 && (norm_whole != 2 || !q_norm), "nv_qk_store: bad norm %d", norm_whole);
+  const bool pairs = !q_norm && norm_whole != 2 && !temp && !bias && !v_first && temp_every == 0 && (rot_dims == 0 || (interleaved && rot_dims <= 256)) &&
                      dim % 4 == 0 && vdim % 4 == 0 && q_off % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 &&
                      proj_row_stride % 4 == 0 && al(proj, 16) && al(q_out, 16) && al(cache, 16);
   QkArgs p{proj, bias, proj_row_stride, q_off, k_off, v_off, q_norm, k_norm, temp, positions, temp_coef, temp_every,
@@ -938,6 +1056,46 @@ extern "C" int nv_qk_rotate_store(const float* proj, const void* bias, int64_t p
     NV_DISPATCH_T(dtype, qk_pairs_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
   else
     NV_DISPATCH_T(dtype, qk_norm_store_kernel<T><<<dim3((unsigned)tokens), dim3(256), 0, (hipStream_t)stream>>>(p));
+  NV_CHECK_LAUNCH();
+  return NV_OK;
+}
+
+// lanes per head of qk_conv_store_kernel
+static int qk_conv_lanes(int dim) {
+  int L = 8;
+  while (4 * L < dim) L *= 2;
+  return L;
+}
+
+extern "C" int nv_qk_conv_store_ok(const void* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off,
+                                   const void* cache, const void* q_out, const void* state, int dim, int vdim, int taps) {
+  auto al = [](const void* q) { return (uintptr_t)q % 16 == 0; };
+  return dim % 4 == 0 && vdim % 4 == 0 && dim <= 256 && taps >= 1 && taps <= QC_MAX_TAPS && q_off % 4 == 0 && k_off % 4 == 0 &&
+         v_off % 4 == 0 && proj_row_stride % 4 == 0 && al(proj) && al(cache) && al(q_out) && al(state);
+}
+
+extern "C" int nv_qk_conv_store(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, const void* w,
+                                int taps, float* state, const int32_t* cu_q, const int32_t* past_lens,
+                                const int32_t* state_slots, const int32_t* seq_of_token, const int32_t* slot_mapping,
+                                void* cache, float* q_out, int64_t tokens, int max_q, int heads, int kv_heads, int dim,
+                                int vdim, int norm, float scale, float eps, int dtype, nv_stream_t stream) {
+  NV_CHECK_ARG(proj && w && cu_q && past_lens && state_slots && seq_of_token && slot_mapping && cache && q_out &&
+                   (state || taps == 1),
+               "nv_qk_conv_store: null pointer");
+  NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_qk_conv_store: bad dtype %d", dtype);
+  NV_CHECK_ARG(tokens >= 0 && heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dim > 0 && vdim > 0,
+               "nv_qk_conv_store: bad shape");
+  NV_CHECK_ARG(nv_qk_conv_store_ok(proj, proj_row_stride, q_off, k_off, v_off, cache, q_out, state, dim, vdim, taps),
+               "nv_qk_conv_store: heads of %d + %d numbers, %d taps or an alignment this launch does not serve", dim, vdim, taps);
+  if (tokens == 0) return NV_OK;
+  const int L = qk_conv_lanes(dim), v_units = (kv_heads * vdim + 4 * L - 1) / (4 * L);
+  const int units = heads + kv_heads + v_units, per = 256 / L, TT = max_q <= 1 ? 1 : 8;
+  QkConvArgs p{proj, proj_row_stride, q_off, k_off, v_off, w, taps, state, cu_q, past_lens, state_slots, seq_of_token,
+               slot_mapping, cache, q_out, tokens, heads, kv_heads, dim, vdim, norm, scale, eps, L, v_units};
+  const dim3 grid((unsigned)((tokens + TT - 1) / TT), (unsigned)((units + per - 1) / per));
+  hipStream_t s = (hipStream_t)stream;
+  if (taps <= 4) NV_DISPATCH_T(dtype, qk_conv_store_kernel<T, 4><<<grid, dim3(256), 0, s>>>(p, TT));
+  else NV_DISPATCH_T(dtype, qk_conv_store_kernel<T, QC_MAX_TAPS><<<grid, dim3(256), 0, s>>>(p, TT));
   NV_CHECK_LAUNCH();
   return NV_OK;
 }

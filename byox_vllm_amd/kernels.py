@@ -440,8 +440,9 @@ EPI_NONE, EPI_GLU, EPI_SOFTCAP, EPI_ROW_GATE, EPI_ACT = 0, 1, 2, 3, 4
 ACT_SILU, ACT_GELU_TANH, ACT_XIELU, ACT_SCALE, ACT_GELU_ERF = 0, 1, 2, 3, 4
 GATE_PER_NUMBER = 1  # EPI_ROW_GATE only (as ``act``): one gate logit per output number instead of one per row and batch
 GLU_CLAMPED = 2      # EPI_GLU only: g sigmoid(1.702 g) (u + 1) with g = min(gate, cap), u = clamp(up, -cap, cap)
-# softmax over the chosen logits / over every expert, renormalised over the chosen / the sigmoid of each chosen logit
-ROUTE_CHOSEN, ROUTE_ALL, ROUTE_SIGMOID = 0, 1, 2
+# softmax over the chosen logits / over every expert, renormalised over the chosen / the sigmoid of each chosen logit /
+# softmax over every expert as it is
+ROUTE_CHOSEN, ROUTE_ALL, ROUTE_SIGMOID, ROUTE_SOFTMAX = 0, 1, 2, 3
 
 
 def _code32(dt) -> int:
@@ -562,18 +563,19 @@ def rms_norm_f32(x, w, eps, out=None):
 
 
 def sandwich_norm(x, y, w_post, w_pre, eps, y_bias=None, rows_idx=None, slot_of=None, weights=None, last_gate=None,
-                  shared=None, shared_gate=None):
+                  shared=None, shared_gate=None, self_rows=None, self_weight=None):
     """fp32 residual rows ``x`` [T, n] take a sublayer's result through its output norm, x += rms_norm(v) * w_post, in
     place; -> rms_norm(x) * w_pre in the weights' dtype (``w_pre`` None: nothing).  v = ``y`` [T, n] + ``y_bias``, or with
     ``slot_of`` int32 [T, C] the sum of f_i * y[slot_of[t, i]] (expert rows; f = ``weights`` [T, C] or 1, the last one
-    sigmoid(``last_gate`` [T]) when given) plus ``shared`` [T, n] times sigmoid(``shared_gate`` [T]).  ``y`` None: the norm
-    alone.  ``rows_idx``: only these rows are normed, and ``x`` is left as it is."""
+    sigmoid(``last_gate`` [T]) when given) plus ``shared`` [T, n] times sigmoid(``shared_gate`` [T]) plus ``self_rows``
+    [T, n] (the model dtype) times ``self_weight`` [T]; a negative slot is skipped.  ``w_post`` None: x += v.  ``y`` None: the
+    norm alone.  ``rows_idx``: only these rows are normed, and ``x`` is left as it is."""
     require_gpu(x, "sandwich_norm")
     T, n = x.shape
     assert x.dtype == torch.float32 and x.is_contiguous()
-    w = w_pre if w_pre is not None else w_post
+    dtype = next((v.dtype for v in (w_pre, w_post, y_bias, self_rows) if v is not None), torch.float32)
     for v in (w_post, w_pre, y_bias):
-        assert v is None or (v.dtype == w.dtype and v.numel() == n and v.is_contiguous())
+        assert v is None or (v.dtype == dtype and v.numel() == n and v.is_contiguous())
     if y is not None:
         assert y.dtype == torch.float32 and y.stride(1) == 1 and y.size(1) == n and (slot_of is not None or y.size(0) == T)
     if slot_of is not None:
@@ -583,14 +585,17 @@ def sandwich_norm(x, y, w_post, w_pre, eps, y_bias=None, rows_idx=None, slot_of=
     for g in (last_gate, shared_gate):
         assert g is None or (g.dtype == torch.float32 and g.dim() == 1 and g.numel() == T)
     assert shared is None or (shared.dtype == torch.float32 and shared.is_contiguous() and shared.shape == (T, n))
+    if self_rows is not None:
+        assert self_rows.dtype == dtype and self_rows.is_contiguous() and self_rows.shape == (T, n)
+        assert self_weight.dtype == torch.float32 and self_weight.is_contiguous() and self_weight.numel() == T
     assert rows_idx is None or rows_idx.dtype == torch.int32
     rows = T if rows_idx is None else rows_idx.numel()
-    out = torch.empty(rows, n, dtype=w.dtype, device=x.device) if w_pre is not None else None
+    out = torch.empty(rows, n, dtype=dtype, device=x.device) if w_pre is not None else None
     check(lib().nv_sandwich_norm(ptr(x), ptr(y), y.stride(0) if y is not None else 0, ptr(y_bias), ptr(w_post), ptr(w_pre),
                                  ptr(out), n, ptr(rows_idx), ptr(slot_of), slot_of.size(1) if slot_of is not None else 0,
                                  ptr(weights), ptr(last_gate), last_gate.stride(0) if last_gate is not None else 0,
                                  ptr(shared), ptr(shared_gate), shared_gate.stride(0) if shared_gate is not None else 0,
-                                 rows, n, eps, _code32(w.dtype), stream()), "nv_sandwich_norm")
+                                 ptr(self_rows), ptr(self_weight), rows, n, eps, _code32(dtype), stream()), "nv_sandwich_norm")
     return out
 
 
@@ -635,11 +640,12 @@ def matrix_memory_state_size(mode, dim, vdim) -> int:
 
 
 def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim, vdim, mode, *, decay=None, bias=None,
-                  gate_offsets=(0, 0), cap=0.0, silu=False, q_scale=1.0, out=None):
+                  gate_offsets=(0, 0), cap=0.0, silu=False, q_scale=1.0, k_scale=1.0, rot=None, out=None):
     """Matrix memory with one decay per head and token over the step's tokens; ``proj`` fp32 [T, *] holds q | k | v at
     ``offsets`` (and, MEM_EXPGATE, one input-gate and one forget-gate logit per head at ``gate_offsets``, to which
-    ``bias`` over proj's columns is added); ``state`` fp32 [slots, heads, state size] is read (unless the request
-    starts) and written back.  -> fp32 [T, heads * vdim]."""
+    ``bias`` over proj's columns is added); ``rot`` fp32 [T, dims]: cosines and sines (rotation_table) by which the first
+    dims numbers of every q and k head turn, i with i + dims / 2; ``state`` fp32 [slots, heads, state size] is read (unless
+    the request starts) and written back.  -> fp32 [T, heads * vdim]."""
     require_gpu(proj, "matrix_memory")
     T = proj.size(0)
     assert proj.dtype == state.dtype == torch.float32 and proj.stride(1) == 1 and state.is_contiguous()
@@ -651,6 +657,8 @@ def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim
     i_off, f_off = gate_offsets
     cols = proj.size(1)
     assert max(q_off + heads * dim, k_off + heads * dim, v_off + heads * vdim) <= cols
+    if rot is not None:
+        assert rot.dtype == torch.float32 and rot.is_contiguous() and rot.size(0) == T and rot.size(1) <= dim
     dt = torch.float32
     if mode == MEM_CONST:
         assert decay is not None and decay.dtype == torch.float32 and decay.numel() == heads and decay.is_cuda
@@ -663,7 +671,19 @@ def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim
     assert out.dtype == torch.float32 and out.stride(1) == 1 and out.size(0) == T and out.size(1) >= heads * vdim
     check(lib().nv_matrix_memory(ptr(proj), proj.stride(0), q_off, k_off, v_off, i_off, f_off, ptr(bias), ptr(decay),
                                  ptr(state), ptr(cu_q), ptr(past_lens), ptr(state_slots), ptr(out), out.stride(0), B, heads,
-                                 dim, vdim, mode, int(silu), q_scale, cap, _code32(dt), stream()), "nv_matrix_memory")
+                                 dim, vdim, mode, int(silu), q_scale, k_scale, ptr(rot), rot.size(1) if rot is not None else 0, cap,
+                                 _code32(dt), stream()), "nv_matrix_memory")
+    return out
+
+
+def rotation_table(positions, inv_freq, out=None):
+    """Cosines, then sines of position * inv_freq (float64 [half]) -> fp32 [T, 2 * half]; the angles are formed in double."""
+    require_gpu(positions, "rotation_table")
+    assert positions.dtype == torch.int64 and positions.is_contiguous()
+    assert inv_freq.dtype == torch.float64 and inv_freq.is_contiguous() and inv_freq.is_cuda
+    T, half = positions.numel(), inv_freq.numel()
+    out = torch.empty(T, 2 * half, dtype=torch.float32, device=positions.device) if out is None else out
+    check(lib().nv_rotation_table(ptr(positions), ptr(inv_freq), ptr(out), T, half, stream()), "nv_rotation_table")
     return out
 
 
@@ -796,13 +816,23 @@ def moe_combine(y, slot_of, weights, shared=None, shared_gate=None, out=None):
     return out
 
 
-def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False):
+def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False, identity=0, correction=None, groups=0, keep_groups=0,
+             scale=1.0, self_weight=None):
     """Routing and ordering of fp32 router logits [T, >= experts].  With ``shared`` every token's last choice is expert
-    number ``experts`` (weight 1): C = top + 1 choices and experts + 1 groups, else C = top.
+    number ``experts`` (weight 1): C = top + 1 choices and experts + 1 groups, else C = top.  The last ``identity`` of the
+    experts + identity router outputs return their input: a choice of one owns no row (its sorted row is -1), and a token's
+    weights of them are summed in ``self_weight`` fp32 [T].  ``correction`` fp32 [experts + identity] is added to the scores
+    where they are compared; ``groups`` > 0: only the ``keep_groups`` best of that many groups of neighbours are chosen from;
+    ``scale`` multiplies the weights.
     -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C], sorted row of every
     choice int32 [T, C], the routed choices' weights fp32 [T, top])."""
     require_gpu(logits, "moe_plan")
-    assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.size(1) >= experts
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.size(1) >= experts + identity
+    assert correction is None or (correction.dtype == torch.float32 and correction.is_contiguous() and correction.is_cuda
+                                  and correction.numel() == experts + identity)
+    assert (identity > 0) == (self_weight is not None)
+    if self_weight is not None:
+        assert self_weight.dtype == torch.float32 and self_weight.is_contiguous() and self_weight.numel() == logits.size(0)
     T, dev, C = logits.size(0), logits.device, top + int(shared)
     idx = torch.empty(T, top, dtype=torch.int32, device=dev)
     weights = torch.empty(T, top, dtype=torch.float32, device=dev)
@@ -810,8 +840,9 @@ def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False):
     sorted_token = torch.empty(T * C, dtype=torch.int32, device=dev)
     sorted_weight = torch.empty(T * C, dtype=torch.float32, device=dev)
     slot_of = torch.empty(T, C, dtype=torch.int32, device=dev)
-    check(lib().nv_moe_plan(ptr(logits), logits.stride(0), T, experts, top, mode, int(shared), ptr(idx), ptr(weights),
-                            ptr(offsets), ptr(sorted_token), ptr(sorted_weight), ptr(slot_of), stream()), "nv_moe_plan")
+    check(lib().nv_moe_plan(ptr(logits), logits.stride(0), T, experts, top, mode, int(shared), identity, ptr(correction), groups,
+                            keep_groups, scale, ptr(idx), ptr(weights), ptr(offsets), ptr(sorted_token), ptr(sorted_weight),
+                            ptr(slot_of), ptr(self_weight), stream()), "nv_moe_plan")
     return offsets, sorted_token, sorted_weight, slot_of, weights
 
 
@@ -867,17 +898,20 @@ def token_shift(h, mu, state, cu_q, past_lens, state_slots, seq_of_token, out=No
     return out
 
 
-def group_rms_norm_f32(x, w, groups, eps, out=None, gate=None):
-    """fp32 rows [T, groups * n]: every part of n numbers by its own root mean square, times w (times sigmoid of the
-    fp32 ``gate`` logits of the same layout, if given) -> rows in w's dtype."""
+def group_rms_norm_f32(x, w, groups, eps, out=None, gate=None, gate_silu=False, out_dtype=None):
+    """fp32 rows [T, groups * n]: every part of n numbers by its own root mean square, times w (None: no weight), times
+    the sigmoid (``gate_silu``: the SiLU) of the fp32 ``gate`` logits of the same layout, if given -> rows in w's dtype
+    (``out_dtype`` where there is no weight)."""
     require_gpu(x, "group_rms_norm_f32")
-    assert x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1 and w.numel() == x.size(1)
-    assert x.size(1) % groups == 0
-    out = torch.empty(x.shape, dtype=w.dtype, device=x.device) if out is None else out
+    assert x.dim() == 2 and x.dtype == torch.float32 and x.stride(1) == 1 and (w is None or w.numel() == x.size(1))
+    assert x.size(1) % groups == 0 and (w is None or out_dtype in (None, w.dtype))
+    dtype = w.dtype if w is not None else out_dtype
+    out = torch.empty(x.shape, dtype=dtype, device=x.device) if out is None else out
+    assert out.dtype == dtype and out.stride(1) == 1 and out.shape == x.shape
     assert gate is None or (gate.dtype == torch.float32 and gate.stride(1) == 1 and gate.shape == x.shape)
     check(lib().nv_group_rmsnorm_f32(ptr(x), x.stride(0), ptr(w), ptr(out), out.stride(0), x.size(0), groups,
                                      x.size(1) // groups, eps, ptr(gate), gate.stride(0) if gate is not None else 0,
-                                     _code32(w.dtype), stream()), "nv_group_rmsnorm_f32")
+                                     int(gate_silu), _code32(dtype), stream()), "nv_group_rmsnorm_f32")
     return out
 
 
@@ -922,11 +956,11 @@ def window_attn(q, cache, block_tables, cu_q, past_lens, seq_of_token, max_q, he
 
 def qk_rotate_store(proj, offsets, positions, scale, slot_mapping, cache, heads, kv_heads, dim, vdim, *, q_norm=None,
                     k_norm=None, eps=0.0, inv_freq=None, rot_dims=0, interleaved=False, mscale=1.0, v_first=None,
-                    vmix=None, bias=None):
+                    vmix=None, bias=None, unit_heads=False):
     """fp32 projections [T, *] with q | k | v at ``offsets`` -> fp32 queries [T, heads * dim] times ``scale``; keys and
     values go to cache rows [G * dim | G * vdim] of ``slot_mapping``.  ``q_norm`` [heads * dim] / ``k_norm``
     [kv_heads * dim]: one RMS norm over all of a token's query numbers (and all of its key numbers) with a weight per
-    number.  ``rot_dims``: the first rot_dims numbers of every head turn by position * inv_freq[i], i with
+    number; ``unit_heads``: every query and key head by its own root mean square, without weights.  ``rot_dims``: the first rot_dims numbers of every head turn by position * inv_freq[i], i with
     i + rot_dims / 2 (``interleaved``: 2i with 2i + 1).  ``v_first`` fp32 [T, G * vdim] (a column slice is fine): the stored values are
     (1 - vmix) v + vmix v_first."""
     require_gpu(proj, "qk_rotate_store")
@@ -938,7 +972,7 @@ def qk_rotate_store(proj, offsets, positions, scale, slot_mapping, cache, heads,
     need = max(q_off + heads * dim, k_off + kv_heads * dim, v_off + kv_heads * vdim)
     assert need <= proj.size(1)
     assert bias is None or (bias.dtype == cache.dtype and bias.is_contiguous() and need <= bias.numel() <= proj.size(1))
-    assert (q_norm is None) == (k_norm is None)
+    assert (q_norm is None) == (k_norm is None) and not (unit_heads and q_norm is not None)
     if q_norm is not None:
         assert q_norm.numel() == heads * dim and k_norm.numel() == kv_heads * dim
         assert q_norm.dtype == k_norm.dtype == cache.dtype and q_norm.is_contiguous() and k_norm.is_contiguous()
@@ -950,11 +984,39 @@ def qk_rotate_store(proj, offsets, positions, scale, slot_mapping, cache, heads,
         assert vmix.dtype == cache.dtype and vmix.numel() == 1 and vmix.is_cuda
     q = torch.empty(T, heads * dim, dtype=torch.float32, device=proj.device)
     check(lib().nv_qk_rotate_store(ptr(proj), ptr(bias), proj.stride(0), q_off, k_off, v_off, ptr(q_norm), ptr(k_norm),
-                                   int(q_norm is not None), None, ptr(positions), 0.0, 0, ptr(inv_freq), int(rot_dims),
+                                   2 if unit_heads else int(q_norm is not None), None, ptr(positions), 0.0, 0, ptr(inv_freq), int(rot_dims),
                                    int(interleaved), float(mscale), ptr(v_first), v_first.stride(0) if v_first is not None else 0,
                                    ptr(vmix) if v_first is not None else None, scale, eps, ptr(slot_mapping), ptr(cache),
                                    ptr(q), T, heads, kv_heads, dim, vdim, _code32(cache.dtype), stream()),
           "nv_qk_rotate_store")
+    return q
+
+
+def qk_conv_store(proj, offsets, w, state, cu_q, past_lens, state_slots, seq_of_token, scale, slot_mapping, cache, heads,
+                  kv_heads, dim, vdim, max_q, *, unit_heads=False, eps=0.0):
+    """fp32 projections [T, *] with q | k | v at ``offsets``, each channel through a causal convolution over time, ``w``
+    [C, taps] over the C channels of q | k | v without bias (``state`` fp32 [slots, taps - 1, C]: a request's last inputs);
+    ``unit_heads``: every query and key head by its root mean square -> fp32 queries [T, heads * dim] times ``scale``;
+    keys and values to the cache rows of ``slot_mapping``.  -> None where the launch does not serve the sizes or
+    alignments at hand: convolve and store in two steps then."""
+    require_gpu(proj, "qk_conv_store")
+    T, B, C = proj.size(0), past_lens.numel(), heads * dim + kv_heads * (dim + vdim)
+    taps = w.size(1)
+    assert proj.dtype == torch.float32 and proj.stride(1) == 1 and w.shape == (C, taps) and w.is_contiguous()
+    assert w.dtype == cache.dtype and cache.is_contiguous() and cache.size(-1) == kv_heads * (dim + vdim)
+    assert taps == 1 or (state.dtype == torch.float32 and state.is_contiguous() and state.shape[1:] == (taps - 1, C))
+    assert cu_q.dtype == past_lens.dtype == state_slots.dtype == seq_of_token.dtype == slot_mapping.dtype == torch.int32
+    assert cu_q.numel() == B + 1 and state_slots.numel() == B and seq_of_token.numel() == slot_mapping.numel() == T
+    q_off, k_off, v_off = offsets
+    assert max(q_off + heads * dim, k_off + kv_heads * dim, v_off + kv_heads * vdim) <= proj.size(1)
+    q = torch.empty(T, heads * dim, dtype=torch.float32, device=proj.device)
+    state_ptr = ptr(state) if taps > 1 else None
+    if not lib().nv_qk_conv_store_ok(ptr(proj), proj.stride(0), q_off, k_off, v_off, ptr(cache), ptr(q), state_ptr, dim, vdim, taps):
+        return None
+    check(lib().nv_qk_conv_store(ptr(proj), proj.stride(0), q_off, k_off, v_off, ptr(w), taps, state_ptr, ptr(cu_q),
+                                 ptr(past_lens), ptr(state_slots), ptr(seq_of_token), ptr(slot_mapping), ptr(cache), ptr(q), T,
+                                 int(max_q), heads, kv_heads, dim, vdim, int(unit_heads), scale, eps, _code32(cache.dtype),
+                                 stream()), "nv_qk_conv_store")
     return q
 
 

@@ -11,7 +11,11 @@ at 0: keep = exp(f + m_(t-1) - m_t), take = exp(i - m_t); a normaliser n_t follo
 o_t = S_t^T q_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6) with q = W_q h / sqrt(dim).  EACH head's o is divided by its own
 root mean square; then weight over all heads, sigmoid(W_g h), projection.
 
-Both read one merged input projection (q | k | v | g [| i | f], then the rows of ``riders``: other consumers of the same
+``Retention``: keep is a constant of the head, take is 1, q and k are rotated by their position (the first ``rot_dims``
+numbers, i with i + rot_dims / 2) and k is scaled by dim^(-1/2); EACH head's o is divided by its own root mean square
+(no weight), multiplied by silu(W_g h) and projected.
+
+All read one merged input projection (q | k | v | g [| i | f], then the rows of ``riders``: other consumers of the same
 input, such as a router beside the mixer) and leave it in fp32: activations, gates, the
 recurrence, the norm and the output gate are fp32.  What a request keeps between steps lives in fp32 slots that the
 engine's StateSlotManager hands out; a request's first tokens start from zero instead of reading the slot.  A mixer whose
@@ -41,7 +45,8 @@ class _MatrixMemoryMixer(nn.Module):
     mode = kernels.MEM_CONST
     extra_shards: tuple = ()
 
-    def __init__(self, width: int, heads: int, dim: int, vdim: int, eps: float, runs: int = 1, riders: dict | None = None):
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, eps: float, runs: int = 1, riders: dict | None = None,
+                 norm_weight: bool = True):
         super().__init__()
         self.heads, self.dim, self.vdim, self.eps = heads, dim, vdim, eps
         shards = {"q": heads * dim, "k": heads * dim, "v": heads * vdim, "g": heads * vdim}
@@ -52,7 +57,10 @@ class _MatrixMemoryMixer(nn.Module):
             self.inp.bias.data.zero_()            # only the gate rows have a bias; the others keep zero
             self.inp.bias.keep_init = True        # ... also under random initialisation
         self.at = {name: self.inp.offset(name) for name in shards}
-        self.norm = nn.Parameter(torch.ones(heads * vdim), requires_grad=False)
+        if norm_weight:
+            self.norm = nn.Parameter(torch.ones(heads * vdim), requires_grad=False)
+        else:
+            self.register_parameter("norm", None)
         self.o = DenseLinear(heads * vdim, width)
         per_head = kernels.matrix_memory_state_size(self.mode, dim, vdim)
         self.runs = [MemoryRun(heads, per_head) for _ in range(runs)]
@@ -60,10 +68,11 @@ class _MatrixMemoryMixer(nn.Module):
     def state_modules(self):
         return list(self.runs)
 
-    def _memory(self, proj, state, ctx):
+    def _memory(self, proj, state, ctx, rot=None):
         raise NotImplementedError
 
     norm_groups = 1
+    gate_silu = False
 
     def project(self, h: torch.Tensor) -> torch.Tensor:
         """The merged input projection, fp32 [T, q | k | v | g | ...]; ``rider(proj, name)`` is a rider's slice of it."""
@@ -73,14 +82,16 @@ class _MatrixMemoryMixer(nn.Module):
         at, rows = self.inp.row_of[name]
         return proj[:, at:at + rows]
 
-    def forward(self, h: torch.Tensor, run: int = 0, positions=None, proj: torch.Tensor | None = None) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, run: int = 0, positions=None, proj: torch.Tensor | None = None,
+                rot: torch.Tensor | None = None) -> torch.Tensor:
         ctx = get_context()
         if proj is None:
             proj = self.project(h)
-        o = self._memory(proj, self.runs[run].state, ctx)
+        o = self._memory(proj, self.runs[run].state, ctx, rot)
         g = self.at["g"]
-        y = kernels.group_rms_norm_f32(o, self.norm.data, self.norm_groups, self.eps,
-                                       gate=proj[:, g:g + self.heads * self.vdim])
+        y = kernels.group_rms_norm_f32(o, self.norm.data if self.norm is not None else None, self.norm_groups, self.eps,
+                                       gate=proj[:, g:g + self.heads * self.vdim], gate_silu=self.gate_silu,
+                                       out_dtype=h.dtype)
         return self.o(y, out_dtype=torch.float32)
 
 
@@ -92,10 +103,27 @@ class LightningAttention(_MatrixMemoryMixer):
         assert len(decay) == heads, f"{len(decay)} decays for {heads} heads"
         self.register_buffer("decay", torch.tensor([float(a) for a in decay], dtype=torch.float32), persistent=False)
 
-    def _memory(self, proj, state, ctx):
+    def _memory(self, proj, state, ctx, rot=None):
         return kernels.matrix_memory(proj, (self.at["q"], self.at["k"], self.at["v"]), state, ctx.cu_seqlens_q,
                                      ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
                                      decay=self.decay, silu=True)
+
+
+class Retention(_MatrixMemoryMixer):
+    mode = kernels.MEM_CONST
+    gate_silu = True
+
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, decay, eps: float, runs: int = 1, riders=None):
+        super().__init__(width, heads, dim, vdim, eps, runs, riders, norm_weight=False)
+        assert len(decay) == heads, f"{len(decay)} decays for {heads} heads"
+        self.norm_groups = heads
+        self.register_buffer("decay", torch.tensor([float(a) for a in decay], dtype=torch.float32), persistent=False)
+
+    def _memory(self, proj, state, ctx, rot=None):
+        """``rot``: the step's cosines and sines (kernels.rotation_table), None where nothing is rotated."""
+        return kernels.matrix_memory(proj, (self.at["q"], self.at["k"], self.at["v"]), state, ctx.cu_seqlens_q,
+                                     ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
+                                     decay=self.decay, k_scale=self.dim ** -0.5, rot=rot)
 
 
 class MLSTM(_MatrixMemoryMixer):
@@ -108,7 +136,7 @@ class MLSTM(_MatrixMemoryMixer):
         self.gate_cap = float(gate_cap)
         self.norm_groups = heads
 
-    def _memory(self, proj, state, ctx):
+    def _memory(self, proj, state, ctx, rot=None):
         return kernels.matrix_memory(proj, (self.at["q"], self.at["k"], self.at["v"]), state, ctx.cu_seqlens_q,
                                      ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
                                      bias=self.inp.bias.data, gate_offsets=(self.at["i"], self.at["f"]),

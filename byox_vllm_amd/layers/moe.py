@@ -1,6 +1,7 @@
 """Feed-forward blocks on nv_linear: the gated unit W_down(act(W_gate h) * (W_up h)) as two launches (gate and up rows
 share one product whose epilogue applies biases, activation and multiplication), a mixture of such units, and a mixture
-of units without a gate (``UnaryMixtureOfExperts``).
+of units without a gate (``UnaryMixtureOfExperts``).  ``GroupedMixtureOfExperts`` chooses within the best groups of
+experts, by corrected scores, and knows experts that return their input.
 
 Mixture: fp32 router logits, the ``top`` largest per token, softmax over the chosen logits only; the (token, choice)
 pairs are ordered by expert on the device, the experts' two products run as grouped launches over the gathered rows
@@ -23,7 +24,8 @@ from byox_vllm_amd.layers.linear import DenseLinear
 from byox_vllm_amd.layers.mlp import UNARY
 
 ACTIVATIONS = {"silu": kernels.ACT_SILU, "gelu_tanh": kernels.ACT_GELU_TANH, "clamped": kernels.GLU_CLAMPED}
-ROUTES = {"chosen": kernels.ROUTE_CHOSEN, "all": kernels.ROUTE_ALL, "sigmoid": kernels.ROUTE_SIGMOID}
+ROUTES = {"chosen": kernels.ROUTE_CHOSEN, "all": kernels.ROUTE_ALL, "sigmoid": kernels.ROUTE_SIGMOID,
+          "softmax": kernels.ROUTE_SOFTMAX}
 
 
 class GatedMLP(nn.Module):
@@ -65,6 +67,15 @@ class MixtureOfExperts(nn.Module):
         at = 0 if part == "gate" else self.ff
         param.data[e, at: at + self.ff].copy_(tensor)
 
+    def expert_rows(self, h, offsets, sorted_token):
+        """The experts' outputs for the (token, choice) pairs ordered by expert, fp32 [T * top, width]."""
+        T, E, top = h.size(0), self.experts, self.top
+        hidden = kernels.linear(h, self.gate_up.data, rows=T * top, a_rows=sorted_token, batch=E,
+                                w_batch_stride=2 * self.ff * self.width, group_offsets=offsets, max_group_rows=T,
+                                epilogue=kernels.EPI_GLU, act=self.act, cap=self.limit)
+        return kernels.linear(hidden, self.down.data, out_dtype=torch.float32, rows=T * top, batch=E,
+                              w_batch_stride=self.width * self.ff, group_offsets=offsets, max_group_rows=T)
+
     def forward(self, h, add=None, logits=None):
         T, E, top = h.size(0), self.experts, self.top
         if logits is None:
@@ -72,15 +83,45 @@ class MixtureOfExperts(nn.Module):
         assert logits.dtype == torch.float32 and logits.shape == (T, E + (1 if self.shared is not None else 0))
         idx, weights = kernels.moe_route(logits, E, top, self.route)
         offsets, sorted_token, slot_of = kernels.moe_sort(idx, E)
-        hidden = kernels.linear(h, self.gate_up.data, rows=T * top, a_rows=sorted_token, batch=E,
-                                w_batch_stride=2 * self.ff * self.width, group_offsets=offsets, max_group_rows=T,
-                                epilogue=kernels.EPI_GLU, act=self.act, cap=self.limit)
-        y = kernels.linear(hidden, self.down.data, out_dtype=torch.float32, rows=T * top, batch=E,
-                           w_batch_stride=self.width * self.ff, group_offsets=offsets, max_group_rows=T)
+        y = self.expert_rows(h, offsets, sorted_token)
         if self.shared is None:
             return kernels.moe_combine(y, slot_of, weights, add)
         assert add is None, "a shared expert and an addend share one input of the combining launch"
         return kernels.moe_combine(y, slot_of, weights, self.shared(h), logits[:, E:])
+
+
+class GroupedMixtureOfExperts(MixtureOfExperts):
+    """Gated experts of which a token uses the ``top`` best of its ``keep`` best groups: the softmax over all router
+    outputs gives scores s; s + correction (one learned number per output) is what is compared, groups of neighbouring
+    outputs by their best member first; a chosen output weighs its expert by scale * s.  The last ``identity`` outputs
+    have no expert: their output is the layer's input.
+
+    The combining step is left to the consumer, as in UnaryMixtureOfExperts: ``forward`` returns the operands of
+    kernels.sandwich_norm, whose launch gathers, weighs and sums the expert rows and adds the identity experts' share."""
+
+    def __init__(self, width: int, experts: int, top: int, ff: int, act: str = "silu", route: str = "softmax",
+                 identity: int = 0, groups: int = 0, keep_groups: int = 0, scale: float = 1.0):
+        super().__init__(width, experts, top, ff, act, route=route, own_router=False)
+        outputs = experts + identity
+        assert groups == 0 or (outputs % groups == 0 and 0 < keep_groups <= groups), \
+            f"{keep_groups} of {groups} groups of {outputs} router outputs"
+        self.identity, self.groups, self.keep_groups, self.scale = identity, groups, keep_groups, float(scale)
+        self.router = DenseLinear(width, outputs)
+        # fp32 whatever the model dtype (16-bit checkpoint values widen exactly)
+        self.correction = nn.Parameter(torch.zeros(outputs, dtype=torch.float32), requires_grad=False)
+
+    def forward(self, h) -> dict:
+        T, E, top = h.size(0), self.experts, self.top
+        logits = self.router(h, out_dtype=torch.float32)
+        self_weight = torch.empty(T, dtype=torch.float32, device=h.device) if self.identity else None
+        offsets, tokens, _, slot_of, weights = kernels.moe_plan(
+            logits, E, top, self.route, identity=self.identity, correction=self.correction.data, groups=self.groups,
+            keep_groups=self.keep_groups, scale=self.scale, self_weight=self_weight)
+        y = self.expert_rows(h, offsets, tokens)
+        result = {"y": y, "slot_of": slot_of, "weights": weights}
+        if self.identity:
+            result.update(self_rows=h, self_weight=self_weight)
+        return result
 
 
 class UnaryMixtureOfExperts(nn.Module):

@@ -13,6 +13,8 @@ runs f and passes (y, gate logits, this module) on as the next pending result.  
 
     x <- x + rms_norm(f(rms_norm(x) * w_pre)) * w_post
 
+``PreNorm`` is the pair without the second norm, x <- x + f(rms_norm(x) * w).
+
 Its update is deferred the same way: ``begin`` takes the PREVIOUS sublayer's result through that sublayer's output norm
 into the residual and norms the new rows for this one, in one launch (csrc/rowops.hip: nv_sandwich_norm)."""
 
@@ -80,11 +82,18 @@ class SandwichNorm(nn.Module):
         """``pending`` = (the previous sublayer's result as keywords of kernels.sandwich_norm, its SandwichNorm) or None.
         -> this sublayer's input in the model dtype (of the rows ``rows_idx`` only, if given: ``x`` then stays as it is)."""
         result, norm = pending if pending is not None else ({"y": None}, None)
-        return kernels.sandwich_norm(x, w_post=norm.post.data if norm is not None else None, w_pre=self.pre.data, eps=self.eps,
-                                     rows_idx=rows_idx, **result)
+        w_post = norm.post.data if norm is not None and norm.post is not None else None
+        return kernels.sandwich_norm(x, w_post=w_post, w_pre=self.pre.data, eps=self.eps, rows_idx=rows_idx, **result)
 
     @staticmethod
     def settle(x: torch.Tensor, pending) -> None:
         """The pending result joins ``x`` (nothing is normed for a next sublayer)."""
         result, norm = pending
-        kernels.sandwich_norm(x, w_post=norm.post.data, w_pre=None, eps=norm.eps, **result)
+        kernels.sandwich_norm(x, w_post=norm.post.data if norm.post is not None else None, w_pre=None, eps=norm.eps, **result)
+
+
+class PreNorm(SandwichNorm):
+    """The norm of a sublayer that is normed on its input only; also the norm behind the last sublayer."""
+
+    def __init__(self, width: int, eps: float):
+        super().__init__(width, eps, final=True)

@@ -12,6 +12,7 @@ _MODELS = {
     "Nonetar": ("byox_vllm_amd.models.nonetar", "NonetarForCausalLM"),
     "Zamusun": ("byox_vllm_amd.models.zamusun", "ZamusunForCausalLM"),
     "Vasonex": ("byox_vllm_amd.models.vasonex", "VasonexForCausalLM"),
+    "Zekazen": ("byox_vllm_amd.models.zekazen", "ZekazenForCausalLM"),
     "Kikelorn": ("byox_vllm_amd.models.kikelorn", "KikelornForCausalLM"),
 }
 DEFAULT = "Qwen3ForCausalLM"

@@ -400,13 +400,14 @@ int nv_gated_postnorm_add_conv(float* x, const float* y, int64_t y_row_stride, c
  * y null: x as it is; w_post null: x += v; w_pre / out null: the residual only.  slot_of [rows, choices] (may be null):
  * v is the sum over i of f_i * y[slot_of[t][i]] (rows of a mixture's experts; f_i = weights[t * choices + i], 1 when
  * weights is null; with last_gate the last choice has f = sigmoid(last_gate[t * last_gate_stride])) plus, when given,
- * shared[t] * sigmoid(shared_gate[t * shared_gate_stride]).  rows_idx: output row i is made from row rows_idx[i] of x and
+ * shared[t] * sigmoid(shared_gate[t * shared_gate_stride]).  A negative slot_of is skipped; with self (rows of the storage
+ * type, identity experts) v also takes self[t] * self_weight[t].  rows_idx: output row i is made from row rows_idx[i] of x and
  * of y's arrays, and x is left as it is. */
 int nv_sandwich_norm(float* x, const float* y, int64_t y_row_stride, const void* y_bias, const void* w_post,
                      const void* w_pre, void* out, int64_t out_row_stride, const int32_t* rows_idx, const int32_t* slot_of,
                      int choices, const float* weights, const float* last_gate, int64_t last_gate_stride,
-                     const float* shared, const float* shared_gate, int64_t shared_gate_stride, int64_t rows, int n,
-                     float eps, int dtype, nv_stream_t stream);
+                     const float* shared, const float* shared_gate, int64_t shared_gate_stride, const void* self,
+                     const float* self_weight, int64_t rows, int n, float eps, int dtype, nv_stream_t stream);
 
 /* RMS norm of fp32 rows: out = x / sqrt(mean(x^2) + eps) * w, rounded to the storage type. */
 int nv_rmsnorm_f32(const float* x, int64_t x_row_stride, const void* w, void* out, int64_t out_row_stride, int64_t rows,
@@ -440,13 +441,18 @@ int nv_gla_recurrent(const float* proj, int64_t proj_row_stride, int q_off, int 
  * numbers per head (the matrix; in mode 1 also normaliser and maximum, one copy per 64 value columns).  mode 0: keep = decay[h], take = 1 (lightning attention); mode 1: exponential gates with a running
  * maximum and a normaliser (the matrix memory of xLSTM): i = cap tanh(zi / cap), f = logsigmoid(cap tanh(zf / cap)) from
  * the logits at columns i_off + h and f_off + h of proj (plus `bias`, a vector over proj's columns in the storage type,
- * may be null), o_t divided by max(|n_t . q_t|, exp(-m_t)) + 1e-6.  silu: q, k and v pass through SiLU first.  out: fp32
- * rows, head h at columns h * vdim. */
+ * may be null), o_t divided by max(|n_t . q_t|, exp(-m_t)) + 1e-6.  silu: q, k and v pass through SiLU first.  rot_dims > 0:
+ * the first rot_dims numbers of every q and k head turn, number i with i + rot_dims / 2, by the cosines and sines in row t
+ * of rot (nv_rotation_table); then q times q_scale and k times k_scale.  out: fp32 rows, head h at columns h * vdim. */
 int64_t nv_matrix_memory_state_size(int mode, int dim, int vdim);
 int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int i_off, int f_off,
                      const void* bias, const float* decay, float* state, const int32_t* cu_q, const int32_t* past_lens,
                      const int32_t* state_slots, float* out, int64_t out_row_stride, int num_seqs, int heads, int dim,
-                     int vdim, int mode, int silu, float q_scale, float cap, int dtype, nv_stream_t stream);
+                     int vdim, int mode, int silu, float q_scale, float k_scale, const float* rot, int rot_dims, float cap,
+                     int dtype, nv_stream_t stream);
+/* out[t] (2 * half fp32 numbers): cosines, then sines of positions[t] * inv_freq[i], formed in double. */
+int nv_rotation_table(const int64_t* positions, const double* inv_freq, float* out, int64_t tokens, int half,
+                      nv_stream_t stream);
 
 /* Latent attention (csrc/latent_attn.hip): cache rows [kv_rank | rot_dim] per token, shared by all heads.  The first
  * rot_dims numbers of the rotated parts turn by positions[t] * inv_freq[i]: dimension i with i + rot_dims / 2, or with
@@ -485,18 +491,24 @@ int nv_latent_attn(const float* qa, const void* cache, const int32_t* block_tabl
 
 /* Mixture of experts (csrc/moe.hip): routing, ordering by expert, weighted combination.  nv_moe_route mode 0: softmax
  * over the chosen logits; 1: softmax over all experts, chosen scores divided by (their sum + 1e-20); 2: the sigmoid of
- * the chosen logits as it is.  nv_moe_plan routes and orders: weights as nv_moe_route's [tokens, top]; with shared = 1
+ * the chosen logits as it is; 3: softmax over all experts as it is.  nv_moe_plan routes and orders: weights as nv_moe_route's [tokens, top]; with shared = 1
  * every token also has choice `top`, expert number `experts` with weight 1, so the arrays cover top + shared choices per
  * token and experts + shared groups; sorted_weight (may be null) is the weight of every sorted row.  Short steps take one
- * launch.  nv_moe_combine
+ * launch.
+ * Its further options: identity router outputs behind the experts stand for experts that return their input (chosen ones
+ * own no rows, slot_of -1; self_weight [tokens] receives the sum of a token's weights of them); correction [experts +
+ * identity] is added to the scores where they are compared, not to the weights; groups > 0: neighbouring outputs form
+ * equal groups and only the keep_groups groups with the largest compared score are chosen from; scale multiplies the
+ * weights (correction and groups: modes 1 - 3).  nv_moe_combine
  * adds `shared` times sigmoid(shared_gate) per token, or `shared` as it is when shared_gate is null. */
 int nv_moe_route(const float* logits, int64_t row_stride, int32_t* idx, float* weights, int64_t tokens, int experts,
                  int top, int mode, nv_stream_t stream);
 int nv_moe_sort(const int32_t* idx, int64_t tokens, int experts, int top, int32_t* offsets, int32_t* sorted_token,
                 int32_t* slot_of, nv_stream_t stream);
 int nv_moe_plan(const float* logits, int64_t row_stride, int64_t tokens, int experts, int top, int mode, int shared,
-                int32_t* idx, float* weights, int32_t* offsets, int32_t* sorted_token, float* sorted_weight,
-                int32_t* slot_of, nv_stream_t stream);
+                int identity, const float* correction, int groups, int keep_groups, float scale, int32_t* idx, float* weights,
+                int32_t* offsets, int32_t* sorted_token, float* sorted_weight, int32_t* slot_of, float* self_weight,
+                nv_stream_t stream);
 int nv_moe_combine(const float* y, const int32_t* slot_of, const float* weights, int top, const float* shared,
                    const float* shared_gate, int64_t shared_gate_stride, float* out, int64_t tokens, int width,
                    nv_stream_t stream);
@@ -511,7 +523,8 @@ int nv_moe_combine(const float* y, const int32_t* slot_of, const float* weights,
  * nv_token_shift: out[t] = h[t] + (h[t-1] - h[t]) * mu; the row before a portion comes from the request's slot of
  *   state [slots, width] (zeros when past_lens is 0), which then receives the portion's last row.
  * nv_group_rmsnorm_f32: fp32 rows of `groups` parts of n numbers, each part divided by its own root mean square, times
- *   w, times sigmoid(gate) when gate logits (fp32 rows of the same layout) are given. */
+ *   w (null: no weight), times sigmoid(gate), or silu(gate) with gate_silu, when gate logits (fp32 rows of the same
+ *   layout) are given. */
 int nv_embed_sinusoid(const int64_t* ids, const int64_t* positions, const void* table, const double* inv_freq, float* out,
                       int64_t tokens, int streams, int width, int64_t vocab, int dtype, nv_stream_t stream);
 int nv_hc_norm(float* x, int streams, int width, const float* delta, int64_t delta_row_stride, const float* hc_prev,
@@ -522,7 +535,7 @@ int nv_token_shift(const float* h, const void* mu, float* state, const int32_t* 
                    int dtype, nv_stream_t stream);
 int nv_group_rmsnorm_f32(const float* x, int64_t x_row_stride, const void* w, void* out, int64_t out_row_stride,
                          int64_t rows, int groups, int n, float eps, const float* gate, int64_t gate_row_stride,
-                         int dtype, nv_stream_t stream);
+                         int gate_silu, int dtype, nv_stream_t stream);
 
 /* ---- softmax attention with shaped scores over a paged cache of rows [k: G * dim | v: G * vdim] (csrc/window_attn.hip) ----
  * nv_qk_norm_store: per-head RMS norm of the fp32 q and k projections plus `bias` (a vector over the projection's columns,
@@ -550,7 +563,8 @@ int nv_window_attn(const float* q, const void* cache, const int32_t* block_table
  *   floor(i / chunk) == floor(j / chunk), positions counted from the sequence's start; keep_first > 0 (not together with
  *   chunk): the sequence's first keep_first keys stay visible to every later query beside its window.
  * nv_qk_rotate_store: nv_qk_store with three more options.  norm_whole: one root mean square over all heads * dim query
- *   numbers (and all kv_heads * dim key numbers), weights [heads * dim] and [kv_heads * dim].  rot_dims > 0: after the
+ *   numbers (and all kv_heads * dim key numbers), weights [heads * dim] and [kv_heads * dim]; norm_whole 2: one per head,
+ *   without weights (q_norm and k_norm null).  rot_dims > 0: after the
  *   norm the first rot_dims numbers of every query and key head are rotated, dimension i with i + rot_dims / 2 (interleaved:
  *   2i with 2i + 1), by the angle positions[t] * inv_freq[i], cosine and sine times mscale.  v_first (fp32 [tokens, v_first_row_stride], may be
  *   null): the stored values are (1 - lam) v + lam v_first with lam = vmix[0] (storage type). */
@@ -570,6 +584,17 @@ int nv_qk_rotate_store(const float* proj, const void* bias, int64_t proj_row_str
                        const float* v_first, int64_t v_first_row_stride, const void* vmix, float scale, float eps,
                        const int32_t* slot_mapping, void* cache, float* q_out, int64_t tokens, int heads, int kv_heads,
                        int dim, int vdim, int dtype, nv_stream_t stream);
+/* nv_qk_conv_store: the store behind a short causal convolution (no bias) over time on every channel of q, k and v; w
+ *   [H dim + G dim + G vdim, taps], state [slots, taps - 1, H dim + G dim + G vdim] keeps the last inputs; norm: every
+ *   query and key head is then divided by its root mean square; q * scale to q_out, k and v to the cache.  Serves what
+ *   nv_qk_conv_store_ok admits (heads of a multiple of 4 numbers, 16-byte aligned arrays, at most 8 taps). */
+int nv_qk_conv_store_ok(const void* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, const void* cache,
+                        const void* q_out, const void* state, int dim, int vdim, int taps);
+int nv_qk_conv_store(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, const void* w, int taps,
+                     float* state, const int32_t* cu_q, const int32_t* past_lens, const int32_t* state_slots,
+                     const int32_t* seq_of_token, const int32_t* slot_mapping, void* cache, float* q_out, int64_t tokens,
+                     int max_q, int heads, int kv_heads, int dim, int vdim, int norm, float scale, float eps, int dtype,
+                     nv_stream_t stream);
 /* Bytes of scratch with which a launch of one token per request (max_q 1) lets several workgroups share a token's
  * keys (their shares are joined by a second kernel); 0 where that does not apply.  Without the scratch (null) the
  * launch keeps one workgroup per token and key/value head. */
