@@ -282,7 +282,7 @@ def run_generate_workload(args):
     print(json.dumps(line), flush=True)
 
 
-# --arch-compare: the Rurutar, Nonetar, Zamusun, Kikelorn and Vasonex designs beside the dense Qwen3 decoder (and beside each
+# --arch-compare: the Rurutar, Nonetar, Zamusun, Kikelorn, Vasonex and Zekazen designs beside the dense Qwen3 decoder (and beside each
 # other) at equal width, depth, active feed-forward size and vocabulary, both through LLM.generate: prefill and decode tokens/s.
 # name: (width, layers, prompts, prompt length, decoded tokens)
 ARCH_COMPARE_SIZES = {
@@ -410,6 +410,26 @@ def vasonex_bench_config(width: int, layers: int, vocab: int = 32000):
     return vasonex_config(raw, dtype=torch.bfloat16)
 
 
+def zekazen_bench_config(width: int, layers: int, vocab: int = 32000):
+    """A Zekazen configuration with the proportions of a real model's layers: retention with 128 x 128 states in turn with
+    attention behind four taps (two query heads per key head of 128, a window of 512); every layer carries 16 experts of
+    1.5 x width and 8 identity outputs in 8 groups, of which a token uses three of the best four groups': on average two
+    experts and one identity, the dense comparator's active feed-forward size."""
+    from byox_vllm_amd.models.zekazen import zekazen_config
+    heads = width // 128
+    kinds = [
+        {"type": "retention", "mixer": {"heads": heads, "dim": 128, "vdim": 128, "rot": {"base": 10000.0, "dims": 128},
+                                        "decay": [1.0 - 2.0 ** -(5 + 5 * h / max(heads - 1, 1)) for h in range(heads)]}},
+        {"type": "attention", "mixer": {"heads": heads, "kv_heads": max(1, heads // 2), "dim": 128, "vdim": 128, "conv": 4,
+                                        "scale": 128 ** -0.5, "mask": {"size": 512}}},
+    ]
+    moe = {"kind": "moe", "router": {"experts": 16, "identity": 8, "top": 3, "groups": {"count": 8, "keep": 4}, "scale": 1.5},
+           "expert": {"ff": 3 * width // 2}}
+    specs = [dict(json.loads(json.dumps(kinds[i % 2])), mlp=moe) for i in range(layers)]
+    raw = {"architecture": "Zekazen", "vocab": vocab, "width": width, "norm": {"eps": 1e-5}, "layers": specs}
+    return zekazen_config(raw, dtype=torch.bfloat16)
+
+
 def run_arch_compare(args):
     from byox_vllm_amd import LLM, SamplingParams
     from byox_vllm_amd.config import qwen2_config
@@ -417,7 +437,8 @@ def run_arch_compare(args):
     random.seed(0)
     results = []
     designs = {"rurutar": rurutar_bench_config, "nonetar": nonetar_bench_config, "zamusun": zamusun_bench_config,
-               "kikelorn": kikelorn_bench_config, "vasonex": vasonex_bench_config}
+               "kikelorn": kikelorn_bench_config, "vasonex": vasonex_bench_config,
+               "zekazen": zekazen_bench_config}
     chosen = [d for d in args.arch_designs.split(",") if d]
     assert chosen and all(d in designs for d in chosen), f"--arch-designs: a subset of {sorted(designs)}"
     for name, (width, layers, num, plen, decoded) in ARCH_COMPARE_SIZES.items():
@@ -542,7 +563,8 @@ def main():
                     help="instead of the decode benchmark: prefill and decode tokens/s of the designs named by --arch-designs "
                          "beside the dense Qwen3 decoder at equal size (one GPU, LLM.generate)")
     ap.add_argument("--arch-designs", default="rurutar",
-                    help="--arch-compare: the designs to run beside the dense decoder, comma-separated (rurutar, nonetar, zamusun, kikelorn, vasonex)")
+                    help="--arch-compare: the designs to run beside the dense decoder, comma-separated (rurutar, nonetar, zamusun, "
+                         "kikelorn, vasonex, zekazen)")
     ap.add_argument("--arch-sizes", default="", help="--arch-compare: comma-separated subset of " + ",".join(ARCH_COMPARE_SIZES))
     args = ap.parse_args()
     if args.arch_compare:

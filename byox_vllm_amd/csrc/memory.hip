@@ -21,6 +21,13 @@
 // sixteen at a time: k and q rows in LDS (padded to DMAX with zeros), the thread's own v values in registers; the gates
 // of the chunk are a scalar recurrence that one thread walks while the others stage.  Thread d < dim also carries n[d];
 // the sixteen n . q meet through wavefront sums.
+//
+// Prompts in the first form take retention_chunk_kernel instead: with ONE constant decay per head, C tokens at once are
+// matrix products on the fp32 matrix cores (v_mfma_f32_16x16x4_f32, true fp32),
+//   o_i = decay^(i+1) S^T q_i + sum_(j <= i) decay^(i-j) (q_i . k_j) v_j,
+//   S  <- decay^n S + sum_j decay^(n-1-j) k_j v_j^T,
+// so a chunk costs three short phases instead of C dependent steps.  Each power of the decay is formed on its own (no
+// quotients of powers: nothing overflows or cancels, however small the decay).
 #include "anyt.h"
 
 namespace {
@@ -287,6 +294,256 @@ __global__ __launch_bounds__(256) void matrix_memory_generic_kernel(MemArgs p) {
     for (int c = 0; c < copies; ++c) n_g[c * (p.dim + 1) + p.dim] = m_run;
 }
 
+// A workgroup of eight wavefronts owns one (head, request, slice of 64 state columns) and walks the request's tokens of this
+// step in chunks of C.  In LDS: the chunk's q and k rows (rotated, scaled), its values and the state TRANSPOSED (column
+// major: the products read four consecutive k numbers of a row or column per access), the decayed scores.  The state itself
+// stays in the wavefronts' accumulators from chunk to chunk; its LDS copy serves the products with q.  Matrix steps of four
+// numbers take the numbers {16 kk + 4 g + m : g = 0 .. 3} of a sum in step m, so one 16-byte access feeds four of them.
+// The next chunk's rows are on their way from memory while a chunk is worked on.
+constexpr int RC_WAVES = 8, RC_COLS = 64;
+
+constexpr size_t rc_lds_floats(int dmax, int c) {
+  return (size_t)(2 * c + RC_COLS) * (dmax + 4) + (size_t)(RC_COLS + c) * (c + 4) + c + 4;
+}
+
+template <int DMAX, int C>
+__global__ __launch_bounds__(64 * RC_WAVES) void retention_chunk_kernel(MemArgs p) {
+  constexpr int DP = DMAX + 4, CP = C + 4, DT = DMAX / 16, CT = C / 16, NTHR = 64 * RC_WAVES;
+  constexpr int UNITS = C * (DMAX / 8) / NTHR, VUNITS = C * (RC_COLS / 4) / NTHR;       // staged pieces per thread
+  constexpr int OT = CT * 4 / RC_WAVES, ST = DT * 4 / RC_WAVES;                         // 16 x 16 tiles per wavefront
+  static_assert(UNITS >= 1 && VUNITS >= 1 && OT >= 1 && ST >= 1 && (ST <= 4 || ST % 4 == 0), "tiles fit the wavefronts");
+  extern __shared__ float4 lds4[];
+  float* sq = reinterpret_cast<float*>(lds4);     // [C][DP]
+  float* sk = sq + C * DP;                        // [C][DP]
+  float* st = sk + C * DP;                        // [64][DP] state, transposed
+  float* sv = st + RC_COLS * DP;                  // [64][CP] values, transposed
+  float* sp = sv + RC_COLS * CP;                  // [C][CP] decayed scores
+  float* pw = sp + C * CP;                        // [C + 1] powers of the decay
+  const int h = blockIdx.x, b = blockIdx.y, col0 = blockIdx.z * RC_COLS;
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, lc = lane & 15, lg = lane >> 4;
+  const int d = p.dim, vd = p.vdim, half = p.rot_dims >> 1;
+  const int t0 = p.cu_q[b], t1 = p.cu_q[b + 1];
+  if (t1 <= t0) return;
+  float* S_g = p.state + ((int64_t)p.slots[b] * p.H + h) * p.per_head;
+  const bool fresh = p.past[b] == 0;
+  for (int i = tid; i <= C; i += NTHR) pw[i] = (float)pow((double)p.decay[h], (double)i);
+
+  // staging: unit u of a token is a pair of four-number pieces of q and k that turn together (or two that do not turn)
+  const f32x4 zero = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  f32x4 q_a[UNITS], q_b[UNITS], k_a[UNITS], k_b[UNITS], cs[UNITS], sn[UNITS], vv[VUNITS];
+  auto places = [&](int i, int& j, int& a, int& c) {
+    const int u = tid + i * NTHR, pu = u % (DMAX / 8);
+    j = u / (DMAX / 8);
+    a = pu * 4 < half ? pu * 4 : p.rot_dims + (pu * 4 - half) * 2;
+    c = pu * 4 < half ? a + half : a + 4;
+  };
+  auto fetch = [&](int c0) {
+    const int n = min(C, t1 - c0);
+#pragma unroll
+    for (int i = 0; i < UNITS; ++i) {
+      int j, a, c;
+      places(i, j, a, c);
+      q_a[i] = q_b[i] = k_a[i] = k_b[i] = cs[i] = sn[i] = zero;
+      if (j < n && a < d) {
+        const float* row = p.proj + (int64_t)(c0 + j) * p.proj_rs + h * d;
+        q_a[i] = *reinterpret_cast<const f32x4*>(row + p.q_off + a);
+        q_b[i] = *reinterpret_cast<const f32x4*>(row + p.q_off + c);
+        k_a[i] = *reinterpret_cast<const f32x4*>(row + p.k_off + a);
+        k_b[i] = *reinterpret_cast<const f32x4*>(row + p.k_off + c);
+        if (a < half) {
+          const float* rot = p.rot + (int64_t)(c0 + j) * p.rot_dims;
+          cs[i] = *reinterpret_cast<const f32x4*>(rot + a);
+          sn[i] = *reinterpret_cast<const f32x4*>(rot + half + a);
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < VUNITS; ++i) {
+      const int u = tid + i * NTHR, j = (u & 15) + 16 * (u / 256), c = col0 + ((u >> 4) & 15) * 4;
+      vv[i] = zero;
+      if (j < n && c < vd) vv[i] = *reinterpret_cast<const f32x4*>(p.proj + (int64_t)(c0 + j) * p.proj_rs + p.v_off + h * vd + c);
+    }
+  };
+  auto store = [&]() {
+#pragma unroll
+    for (int i = 0; i < UNITS; ++i) {
+      int j, a, c;
+      places(i, j, a, c);
+      const bool turn = a < half;
+      if (!turn && c >= DMAX) continue;            // behind the last number of an unpadded row
+      f32x4 qa = q_a[i], qb = q_b[i], ka = k_a[i], kb = k_b[i];
+      if (p.silu) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          qa[e] = silu_f32(qa[e]);
+          qb[e] = silu_f32(qb[e]);
+          ka[e] = silu_f32(ka[e]);
+          kb[e] = silu_f32(kb[e]);
+        }
+      }
+      if (turn) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const float u = qa[e], v = qb[e], x = ka[e], y = kb[e];
+          qa[e] = u * cs[i][e] - v * sn[i][e];
+          qb[e] = v * cs[i][e] + u * sn[i][e];
+          ka[e] = x * cs[i][e] - y * sn[i][e];
+          kb[e] = y * cs[i][e] + x * sn[i][e];
+        }
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        qa[e] *= p.q_scale;
+        qb[e] *= p.q_scale;
+        ka[e] *= p.k_scale;
+        kb[e] *= p.k_scale;
+      }
+      *reinterpret_cast<f32x4*>(sq + j * DP + a) = qa;
+      *reinterpret_cast<f32x4*>(sq + j * DP + c) = qb;
+      *reinterpret_cast<f32x4*>(sk + j * DP + a) = ka;
+      *reinterpret_cast<f32x4*>(sk + j * DP + c) = kb;
+    }
+#pragma unroll
+    for (int i = 0; i < VUNITS; ++i) {
+      const int u = tid + i * NTHR, j = (u & 15) + 16 * (u / 256), c = ((u >> 4) & 15) * 4;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) sv[(c + e) * CP + j] = maybe_silu(vv[i][e], p.silu);
+    }
+  };
+  auto at4 = [](const float* q) { return *reinterpret_cast<const f32x4*>(q); };
+  auto step4 = [](const f32x4& a, const f32x4& x, f32x4 acc) {
+#pragma unroll
+    for (int m = 0; m < 4; ++m) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[m], x[m], acc, 0, 0, 0);
+    return acc;
+  };
+
+  // this wavefront's tiles: outputs (row tile o_row, column tiles o_col ..), state (tiles s0 .. in row-major order of 4 columns)
+  const int o_row = wv * OT / 4, o_col = wv * OT % 4, s0 = wv * ST;
+  f32x4 acc_s[ST];
+#pragma unroll
+  for (int i = 0; i < ST; ++i) {
+    const int row = (s0 + i) / 4 * 16 + lg * 4, c = (s0 + i) % 4 * 16 + lc;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      acc_s[i][r] = (!fresh && row + r < d && col0 + c < vd) ? S_g[(int64_t)(row + r) * vd + col0 + c] : 0.0f;
+    *reinterpret_cast<f32x4*>(st + c * DP + row) = acc_s[i];
+  }
+  fetch(t0);
+  for (int c0 = t0; c0 < t1; c0 += C) {
+    const int n = min(C, t1 - c0), nt = (n + 15) / 16;
+    store();
+    __syncthreads();
+    if (c0 + C < t1) fetch(c0 + C);
+    // scores of the tiles on and below the diagonal, decayed
+    for (int idx = wv; idx < nt * (nt + 1) / 2; idx += RC_WAVES) {
+      int ti = 0;
+      while ((ti + 1) * (ti + 2) / 2 <= idx) ++ti;
+      const int tj = idx - ti * (ti + 1) / 2;
+      f32x4 acc0 = zero, acc1 = zero;
+#pragma unroll
+      for (int kk = 0; kk < DT; kk += 2) {
+        acc0 = step4(at4(sq + (ti * 16 + lc) * DP + kk * 16 + lg * 4), at4(sk + (tj * 16 + lc) * DP + kk * 16 + lg * 4), acc0);
+        acc1 = step4(at4(sq + (ti * 16 + lc) * DP + kk * 16 + 16 + lg * 4), at4(sk + (tj * 16 + lc) * DP + kk * 16 + 16 + lg * 4),
+                     acc1);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = ti * 16 + lg * 4 + r, j = tj * 16 + lc;
+        sp[i * CP + j] = j <= i ? (acc0[r] + acc1[r]) * pw[i - j] : 0.0f;
+      }
+    }
+    // what the state ahead of the chunk contributes
+    f32x4 acc_o[OT];
+#pragma unroll
+    for (int o = 0; o < OT; ++o) acc_o[o] = zero;
+    if (o_row < nt) {
+#pragma unroll
+      for (int kk = 0; kk < DT; ++kk) {
+        const f32x4 a = at4(sq + (o_row * 16 + lc) * DP + kk * 16 + lg * 4);
+#pragma unroll
+        for (int o = 0; o < OT; ++o) acc_o[o] = step4(a, at4(st + ((o_col + o) * 16 + lc) * DP + kk * 16 + lg * 4), acc_o[o]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float f = pw[o_row * 16 + lg * 4 + r + 1];
+#pragma unroll
+        for (int o = 0; o < OT; ++o) acc_o[o][r] *= f;
+      }
+    }
+    __syncthreads();
+    if (o_row < nt) {
+      for (int kk = 0; kk <= o_row; ++kk) {
+        const f32x4 a = at4(sp + (o_row * 16 + lc) * CP + kk * 16 + lg * 4);
+#pragma unroll
+        for (int o = 0; o < OT; ++o) acc_o[o] = step4(a, at4(sv + ((o_col + o) * 16 + lc) * CP + kk * 16 + lg * 4), acc_o[o]);
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = o_row * 16 + lg * 4 + r;
+        if (i >= n) continue;
+        float* orow = p.out + (int64_t)(c0 + i) * p.out_rs + h * vd + col0;
+#pragma unroll
+        for (int o = 0; o < OT; ++o) {
+          const int c = (o_col + o) * 16 + lc;
+          if (col0 + c < vd) orow[c] = acc_o[o][r];
+        }
+      }
+    }
+    // the state behind the chunk
+    const float keep = pw[n];
+#pragma unroll
+    for (int i = 0; i < ST; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc_s[i][r] *= keep;
+    for (int kk = 0; kk < nt; ++kk) {
+      float f[4];
+#pragma unroll
+      for (int m = 0; m < 4; ++m) f[m] = pw[max(n - 1 - (kk * 16 + lg * 4 + m), 0)];       // rows past n are zero
+      constexpr int COLS = ST < 4 ? ST : 4;                        // column tiles that share a piece of k
+      f32x4 x[COLS];
+#pragma unroll
+      for (int c = 0; c < COLS; ++c) x[c] = at4(sv + ((s0 + c) % 4 * 16 + lc) * CP + kk * 16 + lg * 4);
+#pragma unroll
+      for (int rt = 0; rt < ST / COLS; ++rt) {
+        const int row = (s0 / 4 + rt) * 16 + lc;
+        f32x4 a;
+#pragma unroll
+        for (int m = 0; m < 4; ++m) a[m] = sk[(kk * 16 + lg * 4 + m) * DP + row] * f[m];
+#pragma unroll
+        for (int c = 0; c < COLS; ++c) acc_s[rt * COLS + c] = step4(a, x[c], acc_s[rt * COLS + c]);
+      }
+    }
+    if (c0 + C < t1) {
+#pragma unroll
+      for (int i = 0; i < ST; ++i)
+        *reinterpret_cast<f32x4*>(st + ((s0 + i) % 4 * 16 + lc) * DP + (s0 + i) / 4 * 16 + lg * 4) = acc_s[i];
+      __syncthreads();                 // q, k, v and scores of this chunk are no longer read
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < ST; ++i) {
+    const int row = (s0 + i) / 4 * 16 + lg * 4, c = (s0 + i) % 4 * 16 + lc;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (row + r < d && col0 + c < vd) S_g[(int64_t)(row + r) * vd + col0 + c] = acc_s[i][r];
+  }
+}
+
+template <int DMAX, int C>
+hipError_t launch_retention_chunk(const MemArgs& p, dim3 grid, hipStream_t s) {
+  constexpr size_t lds = rc_lds_floats(DMAX, C) * sizeof(float);
+  static_assert(lds <= 160 * 1024, "the chunk fits the LDS");
+  static bool allowed = false;
+  if (!allowed) {
+    const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&retention_chunk_kernel<DMAX, C>),
+                                             hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    if (e != hipSuccess) return e;
+    allowed = true;
+  }
+  retention_chunk_kernel<DMAX, C><<<grid, dim3(64 * RC_WAVES), lds, s>>>(p);
+  return hipGetLastError();
+}
+
 template <typename T, int DMAX, int CS>
 void launch_mem_mode(const MemArgs& p, int mode, dim3 grid, int threads, size_t lds, hipStream_t s) {
   if (mode == MEM_CONST) matrix_memory_kernel<T, DMAX, CS, MEM_CONST><<<grid, dim3(threads), lds, s>>>(p);
@@ -325,7 +582,8 @@ extern "C" int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int 
                                 int f_off, const void* bias, const float* decay, float* state, const int32_t* cu_q,
                                 const int32_t* past_lens, const int32_t* state_slots, float* out, int64_t out_row_stride,
                                 int num_seqs, int heads, int dim, int vdim, int mode, int silu, float q_scale,
-                                float k_scale, const float* rot, int rot_dims, float cap, int dtype, nv_stream_t stream) {
+                                float k_scale, const float* rot, int rot_dims, float cap, int max_q, int dtype,
+                                nv_stream_t stream) {
   NV_CHECK_ARG(proj && state && cu_q && past_lens && state_slots && out, "nv_matrix_memory: null pointer");
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_matrix_memory: bad dtype %d", dtype);
   NV_CHECK_ARG(mode == MEM_CONST || mode == MEM_EXPGATE, "nv_matrix_memory: bad mode %d", mode);
@@ -357,6 +615,22 @@ extern "C" int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int 
   MemArgs p{proj, proj_row_stride, q_off, k_off, v_off, i_off, f_off, bias, decay, state, cu_q, past_lens, state_slots,
             out, out_row_stride, heads, dim, vdim, (int)nv_matrix_memory_state_size(mode, dim, vdim), silu, q_scale, k_scale, cap,
             rot, rot_dims};
+  // prompts with one constant decay per head: chunks on the matrix cores
+  auto al16 = [](const void* q) { return (uintptr_t)q % 16 == 0; };
+  const int vslices = (vdim + RC_COLS - 1) / RC_COLS;
+  if (mode == MEM_CONST && max_q >= MM_TC && dim % 8 == 0 && dim <= 256 && vdim % 4 == 0 && rot_dims % 8 == 0 &&
+      q_off % 4 == 0 && k_off % 4 == 0 && v_off % 4 == 0 && proj_row_stride % 4 == 0 && al16(proj) && al16(rot) &&
+      vslices <= 65535 && getenv("NV_MATRIX_MEMORY_STEPS") == nullptr && getenv("NV_MATRIX_MEMORY_GENERIC") == nullptr) {
+    const dim3 grid(heads, num_seqs, vslices);
+    const hipError_t e = dim <= 64    ? launch_retention_chunk<64, 64>(p, grid, (hipStream_t)stream)
+                         : dim <= 128 ? launch_retention_chunk<128, 64>(p, grid, (hipStream_t)stream)
+                                      : launch_retention_chunk<256, 32>(p, grid, (hipStream_t)stream);
+    if (e != hipSuccess) {
+      nv_set_error("nv_matrix_memory: %s", hipGetErrorString(e));
+      return NV_ERR_LAUNCH;
+    }
+    return NV_OK;
+  }
   if (dmax > 256 || slices > 65535 || getenv("NV_MATRIX_MEMORY_GENERIC") != nullptr) {
     const size_t glds = ((size_t)2 * dim + 4 + 32) * sizeof(float);
     NV_CHECK_ARG(glds <= 64 * 1024, "nv_matrix_memory: keys of %d numbers exceed the LDS", dim);

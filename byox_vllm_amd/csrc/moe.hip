@@ -25,6 +25,8 @@ struct RouteArgs {
   float scale;               // factor on the weights
   // the choice compares scores (kept in LDS, n numbers per wavefront) and not plain logits
   __host__ __device__ bool scored() const { return correction != nullptr || groups > 0; }
+  // numbers of LDS per wavefront
+  __host__ __device__ int lds_words() const { return n <= 128 || scored() ? n + groups : 0; }
 };
 
 // The best of v[0 .. n) that comes after (pv, pe) in descending order, ties to the lower index: taking one after the
@@ -57,11 +59,95 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
+// At most ROUTE_RANKED outputs: a lane owns one or two of them and counts how many come before its own in descending
+// order (ties: the lower index first), which is the place of its choice; nothing is searched for step by step.  ``lds``:
+// n + groups numbers of this wavefront.  -> false, with nothing written, when something is no number.
+constexpr int ROUTE_RANKED = 128;
+
+__device__ __forceinline__ bool route_token_ranked(const float* __restrict__ row, const RouteArgs& p, int32_t* ti, float* tw,
+                                                   float* lds, int lane) {
+  const int n = p.n, top = p.top, mode = p.mode;
+  float z[2], s[2], c[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) z[i] = lane + 64 * i < n ? row[lane + 64 * i] : -INFINITY;
+  const float m = wave_max_valu(fmaxf(z[0], z[1]));
+  float all = 1.0f;
+  if (mode != 2) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) s[i] = lane + 64 * i < n ? expf(z[i] - m) : 0.0f;
+    if (mode != 0) all = wave_sum_valu(s[0] + s[1]);
+#pragma unroll
+    for (int i = 0; i < 2; ++i) s[i] /= all;
+  } else {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) s[i] = sigmoid_f32(z[i]);
+  }
+  const bool scored = p.scored();
+  bool bad = false;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int e = lane + 64 * i;
+    c[i] = -INFINITY;
+    if (e >= n) continue;
+    c[i] = scored ? s[i] + (p.correction ? p.correction[e] : 0.0f) : z[i];
+    bad |= c[i] != c[i];
+    lds[e] = c[i];
+  }
+  if (__any(bad)) return false;
+  wave_lds_fence();
+  if (p.groups > 0 && p.keep < p.groups) {
+    float* best = lds + n;             // [groups] best member of each group
+    const int size = n / p.groups;
+    for (int g = lane; g < p.groups; g += 64) {
+      float b = -INFINITY;
+      for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, lds[e]);
+      best[g] = b;
+    }
+    wave_lds_fence();
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      const int e = lane + 64 * i;
+      if (e >= n) continue;
+      const int g = e / size;
+      const float b = best[g];
+      int before = 0;
+      for (int o = 0; o < p.groups; ++o) before += (best[o] > b || (best[o] == b && o < g)) ? 1 : 0;
+      if (before >= p.keep) {
+        c[i] = -INFINITY;
+        lds[e] = c[i];
+      }
+    }
+    wave_lds_fence();
+  }
+  int rank[2] = {0, 0};
+  const bool two = n > 64;
+  for (int o = 0; o < n; ++o) {
+    const float v = lds[o];
+    rank[0] += (v > c[0] || (v == c[0] && o < lane)) ? 1 : 0;
+    if (two) rank[1] += (v > c[1] || (v == c[1] && o < lane + 64)) ? 1 : 0;
+  }
+  bool in[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) in[i] = lane + 64 * i < n && rank[i] < top;
+  float factor = p.scale;
+  if (mode == 0) factor /= wave_sum_valu((in[0] ? s[0] : 0.0f) + (in[1] ? s[1] : 0.0f));
+  else if (mode == 1) factor /= wave_sum_valu((in[0] ? s[0] : 0.0f) + (in[1] ? s[1] : 0.0f)) + 1e-20f;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    if (!in[i]) continue;
+    ti[rank[i]] = lane + 64 * i;
+    tw[rank[i]] = s[i] * factor;
+  }
+  wave_lds_fence();                    // the next token's scores take this one's place
+  return true;
+}
+
 // One wavefront routes one token.  Choices come out in descending order.  ``lds``: n + groups numbers of this wavefront,
-// used when p.scored().
+// used when p.lds_words() says so.
 __device__ __forceinline__ void route_token(const float* __restrict__ row, const RouteArgs& p, int32_t* ti, float* tw,
                                             float* lds, int lane) {
   const int n = p.n, top = p.top, mode = p.mode;
+  if (n <= ROUTE_RANKED && route_token_ranked(row, p, ti, tw, lds, lane)) return;
   float all = 0.0f, m = 0.0f;
   if (mode == 1 || mode == 3) {
     m = -INFINITY;
@@ -150,11 +236,11 @@ __device__ __forceinline__ void route_token(const float* __restrict__ row, const
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t rs,
                                                         int32_t* __restrict__ idx, float* __restrict__ wt, int64_t T_,
                                                         RouteArgs p) {
-  extern __shared__ float scores[];                                  // 4 x (n + groups) when the choice compares scores
+  extern __shared__ float scores[];                                  // 4 x p.lds_words()
   const int wv = threadIdx.x >> 6;
   const int64_t t = (int64_t)blockIdx.x * 4 + wv;
   if (t >= T_) return;
-  route_token(logits + t * rs, p, idx + t * p.top, wt + t * p.top, scores + wv * (p.n + p.groups), threadIdx.x & 63);
+  route_token(logits + t * rs, p, idx + t * p.top, wt + t * p.top, scores + wv * p.lds_words(), threadIdx.x & 63);
 }
 
 struct SortArgs {
@@ -242,11 +328,11 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(SortArgs p) {
 // routing and ordering of a short step in one launch: sixteen wavefronts route a token each, then sort together
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ logits, int64_t rs, int32_t* idx_out,
                                                         float* wt_out, SortArgs p, RouteArgs r) {
-  extern __shared__ int32_t cnt[];                  // [E] | choices [tokens * top] | their weights | 16 x (n + groups) scores
+  extern __shared__ int32_t cnt[];                  // [E] | choices [tokens * top] | their weights | 16 x r.lds_words()
   int32_t* choice = cnt + p.E;
   const int64_t pairs = p.tokens * p.top;
   float* weight = reinterpret_cast<float*>(choice + pairs);
-  float* scores = weight + pairs + (threadIdx.x >> 6) * (r.n + r.groups);
+  float* scores = weight + pairs + (threadIdx.x >> 6) * r.lds_words();
   for (int e = threadIdx.x; e < p.E; e += blockDim.x) cnt[e] = 0;
   for (int64_t t = threadIdx.x >> 6; t < p.tokens; t += blockDim.x >> 6)
     route_token(logits + t * rs, r, choice + t * p.top, weight + t * p.top, scores, threadIdx.x & 63);
@@ -289,8 +375,9 @@ extern "C" int nv_moe_route(const float* logits, int64_t row_stride, int32_t* id
   NV_CHECK_ARG(tokens >= 0 && experts > 0 && top > 0 && top <= experts, "nv_moe_route: bad shape experts=%d top=%d",
                experts, top);
   if (tokens == 0) return NV_OK;
-  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 0, (hipStream_t)stream>>>(
-      logits, row_stride, idx, weights, tokens, RouteArgs{experts, top, mode, nullptr, 0, 0, 1.0f});
+  const RouteArgs r{experts, top, mode, nullptr, 0, 0, 1.0f};
+  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 4 * r.lds_words() * sizeof(float), (hipStream_t)stream>>>(
+      logits, row_stride, idx, weights, tokens, r);
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
@@ -323,7 +410,7 @@ extern "C" int nv_moe_plan(const float* logits, int64_t row_stride, int64_t toke
   if (tokens == 0) return NV_OK;
   hipStream_t s = (hipStream_t)stream;
   SortArgs p{idx, weights, tokens, experts, top, shared, self_weight, offsets, sorted_token, sorted_weight, slot_of};
-  const size_t scores = r.scored() ? (size_t)(r.n + groups) * sizeof(float) : 0;      // per wavefront
+  const size_t scores = (size_t)r.lds_words() * sizeof(float);      // per wavefront
   const size_t plan_lds = (experts + 2 * tokens * top) * sizeof(int32_t) + 16 * scores;
   if (tokens <= 64 && tokens * top <= 2048 && plan_lds <= 64 * 1024) {
     moe_plan_kernel<<<dim3(1), dim3(1024), plan_lds, s>>>(logits, row_stride, idx, weights, p, r);

@@ -199,6 +199,40 @@ __global__ __launch_bounds__(256) void group_rmsnorm_f32_wave_kernel(const float
   }
 }
 
+// ... and with parts of a multiple of 4 numbers and 16-byte aligned rows: L lanes (a power of two, 4 L >= n) per part, four
+// numbers per lane and access
+template <typename T>
+__global__ __launch_bounds__(256) void group_rmsnorm_f32_vec_kernel(const float* __restrict__ x, int64_t x_rs,
+                                                                    const T* __restrict__ w, T* __restrict__ out,
+                                                                    int64_t out_rs, int64_t parts, int groups, int n, int L,
+                                                                    float eps, const float* __restrict__ gate,
+                                                                    int64_t gate_rs, int gate_silu) {
+  typedef typename Pack4<T>::type P;
+  const int64_t part = (int64_t)blockIdx.x * (256 / L) + threadIdx.x / L;
+  const int j = (threadIdx.x % L) * 4;
+  const bool on = part < parts && j < n;
+  const int64_t t = on ? part / groups : 0;
+  const int64_t col = on ? (part % groups) * n + j : 0;
+  f32x4 v = on ? *reinterpret_cast<const f32x4*>(x + t * x_rs + col) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  f32x4 z = on && gate ? *reinterpret_cast<const f32x4*>(gate + t * gate_rs + col) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  float ss = v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+  for (int o = 1; o < L; o <<= 1) ss += __shfl_xor(ss, o, 64);
+  if (!on) return;
+  const float inv = 1.0f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) v[i] *= inv;
+  if (w) {
+    const f32x4 wv = Pack4<T>::widen(*reinterpret_cast<const P*>(w + col));
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] *= wv[i];
+  }
+  if (gate) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] *= gate_silu ? silu_f32(z[i]) : sigmoid_f32(z[i]);
+  }
+  *reinterpret_cast<P*>(out + t * out_rs + col) = Pack4<T>::narrow(v);
+}
+
 }  // namespace
 
 extern "C" int nv_embed_sinusoid(const int64_t* ids, const int64_t* positions, const void* table, const double* inv_freq,
@@ -263,6 +297,20 @@ extern "C" int nv_group_rmsnorm_f32(const float* x, int64_t x_row_stride, const 
   NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_group_rmsnorm_f32: bad dtype %d", dtype);
   NV_CHECK_ARG(rows >= 0 && n > 0 && groups > 0 && rows * groups < (1ll << 31), "nv_group_rmsnorm_f32: bad shape");
   if (rows == 0) return NV_OK;
+  auto al16 = [](const void* q) { return (uintptr_t)q % 16 == 0; };
+  if (n <= 256 && n % 4 == 0 && al16(x) && al16(w) && al16(out) && al16(gate) && x_row_stride % 4 == 0 &&
+      out_row_stride % 4 == 0 && gate_row_stride % 4 == 0) {
+    const int64_t parts = rows * groups;
+    int L = 8;
+    while (4 * L < n) L *= 2;
+    const int per = 256 / L;
+    NV_DISPATCH_T(dtype, group_rmsnorm_f32_vec_kernel<T><<<dim3((unsigned)((parts + per - 1) / per)), dim3(256), 0,
+                                                           (hipStream_t)stream>>>(
+                             x, x_row_stride, (const T*)w, (T*)out, out_row_stride, parts, groups, n, L, eps, gate,
+                             gate_row_stride, gate_silu));
+    NV_CHECK_LAUNCH();
+    return NV_OK;
+  }
   if (n <= 256 && groups > 1) {
     const int64_t parts = rows * groups;
     NV_DISPATCH_T(dtype, group_rmsnorm_f32_wave_kernel<T><<<dim3((unsigned)((parts + 3) / 4)), dim3(256), 0,

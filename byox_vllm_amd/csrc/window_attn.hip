@@ -245,10 +245,19 @@ __global__ __launch_bounds__(256) void qk_conv_store_kernel(QkConvArgs p, int TT
   const int64_t t_begin = (int64_t)blockIdx.x * TT, t_end = min(p.tokens, t_begin + TT);
   f32x4 wt[MAXT], win[MAXT];        // inside the walk win[MAXT - 1 - m] is the row m tokens back
   const T* w = reinterpret_cast<const T*>(p.w) + (int64_t)ch * taps;
+  if (taps == 4) {                  // wt[MAXT - 1 - m] multiplies the row m tokens back
 #pragma unroll
-  for (int m = 0; m < MAXT; ++m)    // wt[MAXT - 1 - m] multiplies the row m tokens back
+    for (int i = 0; i < 4; ++i) {
+      const f32x4 v = Pack4<T>::widen(*reinterpret_cast<const P*>(w + i * 4));
 #pragma unroll
-    for (int i = 0; i < 4; ++i) wt[MAXT - 1 - m][i] = m < taps ? ld_f32<T>(w + i * taps + keep - m) : 0.0f;
+      for (int m = 0; m < MAXT; ++m) wt[MAXT - 1 - m][i] = m < 4 ? v[3 - (m & 3)] : 0.0f;
+    }
+  } else {
+#pragma unroll
+    for (int m = 0; m < MAXT; ++m)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) wt[MAXT - 1 - m][i] = m < taps ? ld_f32<T>(w + i * taps + keep - m) : 0.0f;
+  }
   auto row = [&](int64_t t) { return *reinterpret_cast<const f32x4*>(p.proj + max(t, (int64_t)0) * p.proj_rs + col); };
   const f32x4 zero = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
   // before the walk the window stands one token earlier
@@ -256,12 +265,19 @@ __global__ __launch_bounds__(256) void qk_conv_store_kernel(QkConvArgs p, int TT
 #pragma unroll
   for (int m = 1; m < MAXT; ++m) win[MAXT - m] = (m <= keep && t_begin - m >= t_first) ? row(t_begin - m) : zero;
   win[0] = zero;
+  int b = 0;
+  int64_t t0 = 0, t1 = 0;           // the request of token t and its tokens of this step
+  f32x4 x_next = row(t_begin);      // a token's row is on the way while the one before it is worked on
   for (int64_t t = t_begin; t < p.tokens; ++t) {
-    const int b = p.seq_of[t];
-    const int64_t t0 = p.cu_q[b];
+    if (t >= t1) {
+      b = p.seq_of[t];
+      t0 = p.cu_q[b];
+      t1 = p.cu_q[b + 1];
+    }
     // past the tile: only the first tokens of a portion that began inside it
     if (t >= t_end && !(t0 >= t_begin && t0 < t_end && t - t0 < keep)) break;
-    const f32x4 x = row(t);
+    const f32x4 x = x_next;
+    if (TT > 1) x_next = row(min(t + 1, p.tokens - 1));
     if (t == t0 && keep > 0) {
       float* slot = p.state + (int64_t)p.slots[b] * keep * C + ch;
       const bool fresh = p.past[b] == 0;
@@ -269,7 +285,7 @@ __global__ __launch_bounds__(256) void qk_conv_store_kernel(QkConvArgs p, int TT
       for (int m = 1; m < MAXT; ++m)       // slot row keep - m holds the input m tokens ahead of the portion
         win[MAXT - m] = (m <= keep && on && !fresh) ? *reinterpret_cast<const f32x4*>(slot + (int64_t)(keep - m) * C) : zero;
       if (on) {
-        const int n = p.cu_q[b + 1] - (int)t0;
+        const int n = (int)(t1 - t0);
 #pragma unroll
         for (int m = 1; m < MAXT; ++m) {   // the new row keep - m: the input m - 1 tokens ahead of the portion's last one
           if (m > keep) continue;

@@ -640,11 +640,12 @@ def matrix_memory_state_size(mode, dim, vdim) -> int:
 
 
 def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim, vdim, mode, *, decay=None, bias=None,
-                  gate_offsets=(0, 0), cap=0.0, silu=False, q_scale=1.0, k_scale=1.0, rot=None, out=None):
+                  gate_offsets=(0, 0), cap=0.0, silu=False, q_scale=1.0, k_scale=1.0, rot=None, max_q=1, out=None):
     """Matrix memory with one decay per head and token over the step's tokens; ``proj`` fp32 [T, *] holds q | k | v at
     ``offsets`` (and, MEM_EXPGATE, one input-gate and one forget-gate logit per head at ``gate_offsets``, to which
     ``bias`` over proj's columns is added); ``rot`` fp32 [T, dims]: cosines and sines (rotation_table) by which the first
-    dims numbers of every q and k head turn, i with i + dims / 2; ``state`` fp32 [slots, heads, state size] is read (unless
+    dims numbers of every q and k head turn, i with i + dims / 2; ``max_q`` bounds the tokens one request brings (MEM_CONST
+    works on prompts in chunks); ``state`` fp32 [slots, heads, state size] is read (unless
     the request starts) and written back.  -> fp32 [T, heads * vdim]."""
     require_gpu(proj, "matrix_memory")
     T = proj.size(0)
@@ -672,7 +673,7 @@ def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim
     check(lib().nv_matrix_memory(ptr(proj), proj.stride(0), q_off, k_off, v_off, i_off, f_off, ptr(bias), ptr(decay),
                                  ptr(state), ptr(cu_q), ptr(past_lens), ptr(state_slots), ptr(out), out.stride(0), B, heads,
                                  dim, vdim, mode, int(silu), q_scale, k_scale, ptr(rot), rot.size(1) if rot is not None else 0, cap,
-                                 _code32(dt), stream()), "nv_matrix_memory")
+                                 int(max_q), _code32(dt), stream()), "nv_matrix_memory")
     return out
 
 

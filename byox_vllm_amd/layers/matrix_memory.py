@@ -106,7 +106,7 @@ class LightningAttention(_MatrixMemoryMixer):
     def _memory(self, proj, state, ctx, rot=None):
         return kernels.matrix_memory(proj, (self.at["q"], self.at["k"], self.at["v"]), state, ctx.cu_seqlens_q,
                                      ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
-                                     decay=self.decay, silu=True)
+                                     decay=self.decay, silu=True, max_q=ctx.max_seqlen_q)
 
 
 class Retention(_MatrixMemoryMixer):
@@ -123,7 +123,8 @@ class Retention(_MatrixMemoryMixer):
         """``rot``: the step's cosines and sines (kernels.rotation_table), None where nothing is rotated."""
         return kernels.matrix_memory(proj, (self.at["q"], self.at["k"], self.at["v"]), state, ctx.cu_seqlens_q,
                                      ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
-                                     decay=self.decay, k_scale=self.dim ** -0.5, rot=rot)
+                                     decay=self.decay, k_scale=self.dim ** -0.5, rot=rot,
+                                     max_q=ctx.max_seqlen_q)
 
 
 class MLSTM(_MatrixMemoryMixer):

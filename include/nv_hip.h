@@ -443,13 +443,14 @@ int nv_gla_recurrent(const float* proj, int64_t proj_row_stride, int q_off, int 
  * the logits at columns i_off + h and f_off + h of proj (plus `bias`, a vector over proj's columns in the storage type,
  * may be null), o_t divided by max(|n_t . q_t|, exp(-m_t)) + 1e-6.  silu: q, k and v pass through SiLU first.  rot_dims > 0:
  * the first rot_dims numbers of every q and k head turn, number i with i + rot_dims / 2, by the cosines and sines in row t
- * of rot (nv_rotation_table); then q times q_scale and k times k_scale.  out: fp32 rows, head h at columns h * vdim. */
+ * of rot (nv_rotation_table); then q times q_scale and k times k_scale.  max_q bounds
+ * the tokens one request brings (1: token by token; prompts in mode 0 are worked on in chunks).  out: fp32 rows, head h at columns h * vdim. */
 int64_t nv_matrix_memory_state_size(int mode, int dim, int vdim);
 int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int i_off, int f_off,
                      const void* bias, const float* decay, float* state, const int32_t* cu_q, const int32_t* past_lens,
                      const int32_t* state_slots, float* out, int64_t out_row_stride, int num_seqs, int heads, int dim,
                      int vdim, int mode, int silu, float q_scale, float k_scale, const float* rot, int rot_dims, float cap,
-                     int dtype, nv_stream_t stream);
+                     int max_q, int dtype, nv_stream_t stream);
 /* out[t] (2 * half fp32 numbers): cosines, then sines of positions[t] * inv_freq[i], formed in double. */
 int nv_rotation_table(const int64_t* positions, const double* inv_freq, float* out, int64_t tokens, int half,
                       nv_stream_t stream);
