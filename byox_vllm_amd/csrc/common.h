@@ -133,24 +133,6 @@ template <int N> __device__ __forceinline__ float lanes_max(float v) {
   return v;
 }
 
-// the same over all 64 lanes
-__device__ __forceinline__ float wave_sum_valu(float v) {
-  float a, b;
-  v = lanes_sum<16>(v);
-  rows_pair16(v, a, b);
-  v = a + b;
-  rows_pair32(v, a, b);
-  return a + b;
-}
-__device__ __forceinline__ float wave_max_valu(float v) {
-  float a, b;
-  v = lanes_max<16>(v);
-  rows_pair16(v, a, b);
-  v = fmaxf(a, b);
-  rows_pair32(v, a, b);
-  return fmaxf(a, b);
-}
-
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

@@ -338,7 +338,8 @@ int launch_tile(const LinArgs& p, int epi, int batch, hipStream_t s) {
 // Up to 64 rows per (group of) product: the launch is bound by how many weight loads are in flight, so the four
 // wavefronts of a workgroup share ONE 16-column tile and split K between them (four times the workgroups of the
 // general kernel, a quarter of the dependent rounds each); the partial sums meet in LDS and wavefront 0 finishes.
-// NSUB = 16-row sub-tiles (1: at most 16 rows, 4: at most 64).
+// NSUB = 16-row sub-tiles (1: at most 16 rows, 4: at most 64).  Grouped products of 17 to 64 rows take NSUB 2 and a second
+// workgroup for rows past the 32nd: a group rarely has so many, and half the registers let twice the loads be in flight.
 template <typename T, typename TO, int EPI, int NSUB>
 __global__ __launch_bounds__(256) void linear_fewrow_kernel(LinArgs p) {
   typedef typename Frag<T>::type F;
@@ -353,6 +354,7 @@ __global__ __launch_bounds__(256) void linear_fewrow_kernel(LinArgs p) {
     lo = p.group_off[z];
     hi = p.group_off[z + 1];
   }
+  lo += (int64_t)blockIdx.y * (16 * NSUB);
   if (lo >= hi) return;
   const int nsub = (int)((hi - lo + 15) / 16 < NSUB ? (hi - lo + 15) / 16 : NSUB);
   const int n0 = blockIdx.x * 16;
@@ -521,6 +523,7 @@ extern "C" int nv_linear_scaled(const void* a, int64_t a_row_stride, const int32
   if (M <= 64 && K >= 256 && (N + 15) / 16 <= 1048576) {
     dim3 g16((unsigned)((N + 15) / 16), 1, (unsigned)batch);
     if (M <= 16) launch_fewrow_any<1>(p, epilogue, g16, dtype, out_dtype, s);
+    else if (group_offsets) launch_fewrow_any<2>(p, epilogue, dim3(g16.x, (unsigned)((M + 31) / 32), g16.z), dtype, out_dtype, s);
     else launch_fewrow_any<4>(p, epilogue, g16, dtype, out_dtype, s);
     NV_CHECK_LAUNCH();
     return NV_OK;

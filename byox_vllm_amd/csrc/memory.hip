@@ -370,7 +370,6 @@ __global__ __launch_bounds__(64 * RC_WAVES) void retention_chunk_kernel(MemArgs 
       int j, a, c;
       places(i, j, a, c);
       const bool turn = a < half;
-      if (!turn && c >= DMAX) continue;            // behind the last number of an unpadded row
       f32x4 qa = q_a[i], qb = q_b[i], ka = k_a[i], kb = k_b[i];
       if (p.silu) {
 #pragma unroll

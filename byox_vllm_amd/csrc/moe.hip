@@ -11,6 +11,8 @@
 //                    take part in everything but own no rows, a token's weights of them are summed instead
 //   nv_moe_combine : weighted sum of a token's expert rows (+ a sigmoid-gated shared expert)
 // The sum over a token's experts runs in the order of its choices, so it does not depend on what else is in the batch.
+#include <type_traits>
+
 #include "anyt.h"
 
 namespace {
@@ -25,8 +27,9 @@ struct RouteArgs {
   float scale;               // factor on the weights
   // the choice compares scores (kept in LDS, n numbers per wavefront) and not plain logits
   __host__ __device__ bool scored() const { return correction != nullptr || groups > 0; }
-  // numbers of LDS per wavefront
-  __host__ __device__ int lds_words() const { return n <= 128 || scored() ? n + groups : 0; }
+  // numbers of LDS per wavefront: scores, then best members of the groups, each padded to whole 16 bytes
+  __host__ __device__ int n4() const { return (n + 3) & ~3; }
+  __host__ __device__ int lds_words() const { return n <= 128 || scored() ? n4() + ((groups + 3) & ~3) : 0; }
 };
 
 // The best of v[0 .. n) that comes after (pv, pe) in descending order, ties to the lower index: taking one after the
@@ -59,95 +62,142 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
-// At most ROUTE_RANKED outputs: a lane owns one or two of them and counts how many come before its own in descending
-// order (ties: the lower index first), which is the place of its choice; nothing is searched for step by step.  ``lds``:
-// n + groups numbers of this wavefront.  -> false, with nothing written, when something is no number.
+// At most ROUTE_RANKED outputs: a lane owns one of them (of more than 64: two) and counts how many come before its own in
+// descending order (ties: the lower index first), which is the place of its choice; nothing is searched for step by step.
+// LP lanes serve a token, 64 / LP tokens share a wavefront (LP 128: 64 lanes with two outputs each).  ``lds``: p.lds_words()
+// numbers of this token.  What is no number is compared as -inf, so the places are always a permutation.  Every lane of the
+// wavefront takes part; with live == false nothing is read or written.
 constexpr int ROUTE_RANKED = 128;
 
-__device__ __forceinline__ bool route_token_ranked(const float* __restrict__ row, const RouteArgs& p, int32_t* ti, float* tw,
-                                                   float* lds, int lane) {
+// how many of v[0 .. n) come before (x, at) in descending order; v is padded with -inf to whole 16 bytes
+__device__ __forceinline__ int count_before(const float* v, int n, float x, int at) {
+  int before = 0;
+#pragma unroll 2
+  for (int o = 0; o < n; o += 4) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(v + o);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) before += (a[i] > x || (a[i] == x && o + i < at)) ? 1 : 0;
+  }
+  return before;
+}
+
+template <int LP> __device__ __forceinline__ float token_sum(float v) {
+  float a, b;
+  v = lanes_sum<16>(v);
+  if constexpr (LP >= 32) {
+    rows_pair16(v, a, b);
+    v = a + b;
+  }
+  if constexpr (LP >= 64) {
+    rows_pair32(v, a, b);
+    v = a + b;
+  }
+  return v;
+}
+template <int LP> __device__ __forceinline__ float token_max(float v) {
+  float a, b;
+  v = lanes_max<16>(v);
+  if constexpr (LP >= 32) {
+    rows_pair16(v, a, b);
+    v = fmaxf(a, b);
+  }
+  if constexpr (LP >= 64) {
+    rows_pair32(v, a, b);
+    v = fmaxf(a, b);
+  }
+  return v;
+}
+
+template <int LP>
+__device__ __forceinline__ void route_token_ranked(const float* __restrict__ row, bool live, const RouteArgs& p, int32_t* ti,
+                                                   float* tw, float* lds, int lane) {
+  constexpr int W = LP < 64 ? LP : 64, NV = LP / W;
   const int n = p.n, top = p.top, mode = p.mode;
-  float z[2], s[2], c[2];
+  float z[NV], s[NV], c[NV];
 #pragma unroll
-  for (int i = 0; i < 2; ++i) z[i] = lane + 64 * i < n ? row[lane + 64 * i] : -INFINITY;
-  const float m = wave_max_valu(fmaxf(z[0], z[1]));
+  for (int i = 0; i < NV; ++i) {
+    z[i] = live && lane + W * i < n ? row[lane + W * i] : -INFINITY;
+    if (z[i] != z[i]) z[i] = -INFINITY;
+  }
   float all = 1.0f;
-  if (mode != 2) {
+  if (mode == 2) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) s[i] = lane + 64 * i < n ? expf(z[i] - m) : 0.0f;
-    if (mode != 0) all = wave_sum_valu(s[0] + s[1]);
-#pragma unroll
-    for (int i = 0; i < 2; ++i) s[i] /= all;
+    for (int i = 0; i < NV; ++i) s[i] = sigmoid_f32(z[i]);
   } else {
+    float m = z[0];
+    if constexpr (NV == 2) m = fmaxf(z[0], z[1]);
+    m = token_max<LP>(m);
+    float sum = 0.0f;
 #pragma unroll
-    for (int i = 0; i < 2; ++i) s[i] = sigmoid_f32(z[i]);
+    for (int i = 0; i < NV; ++i) {
+      s[i] = lane + W * i < n ? expf(z[i] - m) : 0.0f;
+      sum += s[i];
+    }
+    if (mode != 0) {
+      all = 1.0f / token_sum<LP>(sum);
+#pragma unroll
+      for (int i = 0; i < NV; ++i) s[i] *= all;
+    }
   }
   const bool scored = p.scored();
-  bool bad = false;
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int e = lane + 64 * i;
-    c[i] = -INFINITY;
-    if (e >= n) continue;
-    c[i] = scored ? s[i] + (p.correction ? p.correction[e] : 0.0f) : z[i];
-    bad |= c[i] != c[i];
-    lds[e] = c[i];
+  for (int i = 0; i < NV; ++i) {
+    const int e = lane + W * i;
+    c[i] = z[i];
+    if (scored) {
+      c[i] = s[i] + (p.correction && e < n ? p.correction[e] : 0.0f);
+      if (e >= n || c[i] != c[i]) c[i] = -INFINITY;
+    }
+    if (live && e < p.n4()) lds[e] = c[i];
   }
-  if (__any(bad)) return false;
   wave_lds_fence();
   if (p.groups > 0 && p.keep < p.groups) {
-    float* best = lds + n;             // [groups] best member of each group
+    float* best = lds + p.n4();        // [groups] best member of each group
     const int size = n / p.groups;
-    for (int g = lane; g < p.groups; g += 64) {
+    for (int g = lane; live && g < ((p.groups + 3) & ~3); g += W) {
       float b = -INFINITY;
-      for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, lds[e]);
+      if (g < p.groups) {
+#pragma unroll 4
+        for (int e = g * size; e < (g + 1) * size; ++e) b = fmaxf(b, lds[e]);
+      }
       best[g] = b;
     }
     wave_lds_fence();
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
-      const int e = lane + 64 * i;
-      if (e >= n) continue;
+    for (int i = 0; i < NV; ++i) {
+      const int e = lane + W * i;
+      if (!live || e >= n) continue;
       const int g = e / size;
-      const float b = best[g];
-      int before = 0;
-      for (int o = 0; o < p.groups; ++o) before += (best[o] > b || (best[o] == b && o < g)) ? 1 : 0;
-      if (before >= p.keep) {
+      if (count_before(best, p.groups, best[g], g) >= p.keep) {
         c[i] = -INFINITY;
         lds[e] = c[i];
       }
     }
     wave_lds_fence();
   }
-  int rank[2] = {0, 0};
-  const bool two = n > 64;
-  for (int o = 0; o < n; ++o) {
-    const float v = lds[o];
-    rank[0] += (v > c[0] || (v == c[0] && o < lane)) ? 1 : 0;
-    if (two) rank[1] += (v > c[1] || (v == c[1] && o < lane + 64)) ? 1 : 0;
+  float chosen = 0.0f;
+  int rank[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    rank[i] = live && lane + W * i < n ? count_before(lds, n, c[i], lane + W * i) : top;
+    if (rank[i] < top) chosen += s[i];
   }
-  bool in[2];
-#pragma unroll
-  for (int i = 0; i < 2; ++i) in[i] = lane + 64 * i < n && rank[i] < top;
   float factor = p.scale;
-  if (mode == 0) factor /= wave_sum_valu((in[0] ? s[0] : 0.0f) + (in[1] ? s[1] : 0.0f));
-  else if (mode == 1) factor /= wave_sum_valu((in[0] ? s[0] : 0.0f) + (in[1] ? s[1] : 0.0f)) + 1e-20f;
+  if (mode <= 1) factor /= token_sum<LP>(chosen) + (mode == 1 ? 1e-20f : 0.0f);
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    if (!in[i]) continue;
-    ti[rank[i]] = lane + 64 * i;
+  for (int i = 0; i < NV; ++i) {
+    if (rank[i] >= top) continue;
+    ti[rank[i]] = lane + W * i;
     tw[rank[i]] = s[i] * factor;
   }
   wave_lds_fence();                    // the next token's scores take this one's place
-  return true;
 }
 
-// One wavefront routes one token.  Choices come out in descending order.  ``lds``: n + groups numbers of this wavefront,
-// used when p.lds_words() says so.
+// Any number of outputs: one wavefront routes one token, one choice after the other in descending order.  ``lds``:
+// p.lds_words() numbers of this wavefront.
 __device__ __forceinline__ void route_token(const float* __restrict__ row, const RouteArgs& p, int32_t* ti, float* tw,
                                             float* lds, int lane) {
   const int n = p.n, top = p.top, mode = p.mode;
-  if (n <= ROUTE_RANKED && route_token_ranked(row, p, ti, tw, lds, lane)) return;
   float all = 0.0f, m = 0.0f;
   if (mode == 1 || mode == 3) {
     m = -INFINITY;
@@ -159,7 +209,7 @@ __device__ __forceinline__ void route_token(const float* __restrict__ row, const
   const float* compare = row;
   const bool scored = p.scored();
   if (scored) {
-    float* best = lds + n;           // [groups] best member of each group
+    float* best = lds + p.n4();      // [groups] best member of each group
     for (int e = lane; e < n; e += 64) {
       const float s = mode == 2 ? sigmoid_f32(row[e]) : expf(row[e] - m) / all;
       lds[e] = s + (p.correction ? p.correction[e] : 0.0f);
@@ -233,14 +283,31 @@ __device__ __forceinline__ void route_token(const float* __restrict__ row, const
   for (int j = 0; j < top; ++j) tw[j] = tw[j] / sum * p.scale;
 }
 
+// the wavefront's tokens t0 .. t0 + tokens_per_wave<LP>() - 1; LP 0: by search
+template <int LP> __host__ __device__ constexpr int tokens_per_wave() { return LP > 0 && LP < 64 ? 64 / LP : 1; }
+
+template <int LP>
+__device__ __forceinline__ void route_wave(const float* logits, int64_t rs, int64_t t0, int64_t tokens, const RouteArgs& p,
+                                           int32_t* ti, float* tw, float* lds, int lane) {
+  if constexpr (LP == 0) {
+    route_token(logits + t0 * rs, p, ti + t0 * p.top, tw + t0 * p.top, lds, lane);
+  } else {
+    constexpr int W = LP < 64 ? LP : 64;
+    const int64_t t = t0 + lane / W;
+    route_token_ranked<LP>(logits + t * rs, t < tokens, p, ti + t * p.top, tw + t * p.top, lds + lane / W * p.lds_words(), lane % W);
+  }
+}
+
+template <int LP>
 __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, int64_t rs,
                                                         int32_t* __restrict__ idx, float* __restrict__ wt, int64_t T_,
                                                         RouteArgs p) {
-  extern __shared__ float scores[];                                  // 4 x p.lds_words()
+  extern __shared__ float4 lds4[];                                   // p.lds_words() per token
+  constexpr int TW = tokens_per_wave<LP>();
   const int wv = threadIdx.x >> 6;
-  const int64_t t = (int64_t)blockIdx.x * 4 + wv;
+  const int64_t t = ((int64_t)blockIdx.x * 4 + wv) * TW;
   if (t >= T_) return;
-  route_token(logits + t * rs, p, idx + t * p.top, wt + t * p.top, scores + wv * p.lds_words(), threadIdx.x & 63);
+  route_wave<LP>(logits, rs, t, T_, p, idx, wt, reinterpret_cast<float*>(lds4) + wv * TW * p.lds_words(), threadIdx.x & 63);
 }
 
 struct SortArgs {
@@ -282,62 +349,84 @@ __device__ __forceinline__ void counts_to_starts(int32_t* cnt, const SortArgs& p
 
 // the (token, choice) pairs go to their expert's next free place; idx may be a copy in LDS
 __device__ __forceinline__ void scatter_pairs(int32_t* cnt, const int32_t* idx, const SortArgs& p) {
-  const int64_t pairs = p.tokens * p.top;
+  const int tokens = (int)p.tokens, pairs = tokens * p.top;        // fit 32 bits, checked by the launcher
   const int C = p.top + p.shared;
   if (p.self_weight) {
-    for (int64_t t = threadIdx.x; t < p.tokens; t += blockDim.x) {
+    for (int t = threadIdx.x; t < tokens; t += blockDim.x) {
       float w = 0.0f;
       for (int j = 0; j < p.top; ++j)
         if (idx[t * p.top + j] >= p.E) w += p.wt[t * p.top + j];
       p.self_weight[t] = w;
     }
   }
-  for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x) {
-    if (idx[i] >= p.E) {
-      p.slot_of[i / p.top * C + i % p.top] = -1;
-      continue;
+  constexpr int AHEAD = 8;             // pairs of a thread whose loads, then counters, are on their way together
+  for (int base = threadIdx.x; base < pairs; base += AHEAD * blockDim.x) {
+    int e[AHEAD], slot[AHEAD];
+    float w[AHEAD];
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) {
+      const int i = base + k * blockDim.x;
+      e[k] = i < pairs ? idx[i] : p.E;
+      w[k] = i < pairs && p.sorted_weight ? p.wt[i] : 0.0f;
     }
-    const int slot = atomicAdd(&cnt[idx[i]], 1);
-    p.sorted_token[slot] = (int32_t)(i / p.top);
-    if (p.sorted_weight) p.sorted_weight[slot] = p.wt[i];
-    p.slot_of[i / p.top * C + i % p.top] = slot;
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) slot[k] = e[k] < p.E ? atomicAdd(&cnt[e[k]], 1) : -1;
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) {
+      const int i = base + k * blockDim.x, t = i / p.top;
+      if (i >= pairs) break;
+      p.slot_of[t * C + (i - t * p.top)] = slot[k];
+      if (slot[k] < 0) continue;
+      p.sorted_token[slot[k]] = t;
+      if (p.sorted_weight) p.sorted_weight[slot[k]] = w[k];
+    }
   }
   if (!p.shared) return;
-  const int64_t routed = p.offsets[p.E];             // written before the barrier ahead of this call
-  for (int64_t t = threadIdx.x; t < p.tokens; t += blockDim.x) {
-    const int64_t slot = routed + t;
-    p.sorted_token[slot] = (int32_t)t;
+  const int routed = p.offsets[p.E];                 // written before the barrier ahead of this call
+  for (int t = threadIdx.x; t < tokens; t += blockDim.x) {
+    const int slot = routed + t;
+    p.sorted_token[slot] = t;
     if (p.sorted_weight) p.sorted_weight[slot] = 1.0f;
-    p.slot_of[t * C + p.top] = (int32_t)slot;
+    p.slot_of[t * C + p.top] = slot;
   }
 }
 
 __global__ __launch_bounds__(1024) void moe_sort_kernel(SortArgs p) {
   extern __shared__ int32_t cnt[];   // [E] counts, then cursors
-  const int64_t pairs = p.tokens * p.top;
+  const int pairs = (int)(p.tokens * p.top);
   for (int e = threadIdx.x; e < p.E; e += blockDim.x) cnt[e] = 0;
   __syncthreads();
-  for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x)
-    if (p.idx[i] < p.E) atomicAdd(&cnt[p.idx[i]], 1);
+  for (int base = threadIdx.x; base < pairs; base += 8 * blockDim.x) {
+    int e[8];
+#pragma unroll
+    for (int k = 0; k < 8; ++k) e[k] = base + k * blockDim.x < pairs ? p.idx[base + k * blockDim.x] : p.E;
+#pragma unroll
+    for (int k = 0; k < 8; ++k)
+      if (e[k] < p.E) atomicAdd(&cnt[e[k]], 1);
+  }
   __syncthreads();
   counts_to_starts(cnt, p);
   __syncthreads();
   scatter_pairs(cnt, p.idx, p);
 }
 
-// routing and ordering of a short step in one launch: sixteen wavefronts route a token each, then sort together
+// routing and ordering of a short step in one launch: sixteen wavefronts route the tokens, then sort together
+template <int LP>
 __global__ __launch_bounds__(1024) void moe_plan_kernel(const float* __restrict__ logits, int64_t rs, int32_t* idx_out,
                                                         float* wt_out, SortArgs p, RouteArgs r) {
-  extern __shared__ int32_t cnt[];                  // [E] | choices [tokens * top] | their weights | 16 x r.lds_words()
+  constexpr int TW = tokens_per_wave<LP>();
+  extern __shared__ float4 lds4[];                  // 16 x TW x r.lds_words() | [E] | choices [tokens * top] | their weights
+  const int wv = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  float* scores = reinterpret_cast<float*>(lds4) + wv * TW * r.lds_words();
+  int32_t* cnt = reinterpret_cast<int32_t*>(lds4) + 16 * TW * r.lds_words();
   int32_t* choice = cnt + p.E;
-  const int64_t pairs = p.tokens * p.top;
+  const int tokens = (int)p.tokens, pairs = tokens * p.top;
   float* weight = reinterpret_cast<float*>(choice + pairs);
-  float* scores = weight + pairs + (threadIdx.x >> 6) * r.lds_words();
   for (int e = threadIdx.x; e < p.E; e += blockDim.x) cnt[e] = 0;
-  for (int64_t t = threadIdx.x >> 6; t < p.tokens; t += blockDim.x >> 6)
-    route_token(logits + t * rs, r, choice + t * p.top, weight + t * p.top, scores, threadIdx.x & 63);
+#pragma unroll 1
+  for (int t = wv * TW; t < tokens; t += 16 * TW) route_wave<LP>(logits, rs, t, tokens, r, choice, weight, scores, lane);
   __syncthreads();
-  for (int64_t i = threadIdx.x; i < pairs; i += blockDim.x) {
+  for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
     if (choice[i] < p.E) atomicAdd(&cnt[choice[i]], 1);
     idx_out[i] = choice[i];
     wt_out[i] = weight[i];
@@ -366,6 +455,24 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(const float* __restric
   }
 }
 
+// the kernels' lanes per token for n outputs
+template <typename F>
+void with_lanes(int n, F f) {
+  if (n <= 16) f(std::integral_constant<int, 16>());
+  else if (n <= 32) f(std::integral_constant<int, 32>());
+  else if (n <= 64) f(std::integral_constant<int, 64>());
+  else if (n <= ROUTE_RANKED) f(std::integral_constant<int, 128>());
+  else f(std::integral_constant<int, 0>());
+}
+
+void launch_route(const float* logits, int64_t rs, int32_t* idx, float* weights, int64_t tokens, const RouteArgs& r, hipStream_t s) {
+  with_lanes(r.n, [&](auto lp) {
+    constexpr int LP = decltype(lp)::value, per = 4 * tokens_per_wave<LP>();
+    moe_route_kernel<LP><<<dim3((unsigned)((tokens + per - 1) / per)), dim3(256), per * r.lds_words() * sizeof(float), s>>>(
+        logits, rs, idx, weights, tokens, r);
+  });
+}
+
 }  // namespace
 
 extern "C" int nv_moe_route(const float* logits, int64_t row_stride, int32_t* idx, float* weights, int64_t tokens,
@@ -376,8 +483,7 @@ extern "C" int nv_moe_route(const float* logits, int64_t row_stride, int32_t* id
                experts, top);
   if (tokens == 0) return NV_OK;
   const RouteArgs r{experts, top, mode, nullptr, 0, 0, 1.0f};
-  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 4 * r.lds_words() * sizeof(float), (hipStream_t)stream>>>(
-      logits, row_stride, idx, weights, tokens, r);
+  launch_route(logits, row_stride, idx, weights, tokens, r, (hipStream_t)stream);
   NV_CHECK_LAUNCH();
   return NV_OK;
 }
@@ -385,7 +491,8 @@ extern "C" int nv_moe_route(const float* logits, int64_t row_stride, int32_t* id
 extern "C" int nv_moe_sort(const int32_t* idx, int64_t tokens, int experts, int top, int32_t* offsets,
                            int32_t* sorted_token, int32_t* slot_of, nv_stream_t stream) {
   NV_CHECK_ARG(idx && offsets && sorted_token && slot_of, "nv_moe_sort: null pointer");
-  NV_CHECK_ARG(tokens >= 0 && experts > 0 && experts <= 8192 && top > 0, "nv_moe_sort: bad shape");
+  NV_CHECK_ARG(tokens >= 0 && experts > 0 && experts <= 8192 && top > 0 && tokens * (top + 1) < (1ll << 31),
+               "nv_moe_sort: bad shape");
   SortArgs p{idx, nullptr, tokens, experts, top, 0, nullptr, offsets, sorted_token, nullptr, slot_of};
   moe_sort_kernel<<<dim3(1), dim3(1024), (size_t)experts * sizeof(int32_t), (hipStream_t)stream>>>(p);
   NV_CHECK_LAUNCH();
@@ -410,15 +517,23 @@ extern "C" int nv_moe_plan(const float* logits, int64_t row_stride, int64_t toke
   if (tokens == 0) return NV_OK;
   hipStream_t s = (hipStream_t)stream;
   SortArgs p{idx, weights, tokens, experts, top, shared, self_weight, offsets, sorted_token, sorted_weight, slot_of};
-  const size_t scores = (size_t)r.lds_words() * sizeof(float);      // per wavefront
-  const size_t plan_lds = (experts + 2 * tokens * top) * sizeof(int32_t) + 16 * scores;
-  if (tokens <= 64 && tokens * top <= 2048 && plan_lds <= 64 * 1024) {
-    moe_plan_kernel<<<dim3(1), dim3(1024), plan_lds, s>>>(logits, row_stride, idx, weights, p, r);
+  const size_t scores = (size_t)r.lds_words() * sizeof(float);      // per token that a wavefront works on
+  bool done = false;
+  if (tokens <= 64 && tokens * top <= 2048) {
+    with_lanes(r.n, [&](auto lp) {
+      constexpr int LP = decltype(lp)::value;
+      const size_t lds = (experts + 2 * tokens * top) * sizeof(int32_t) + 16 * tokens_per_wave<LP>() * scores;
+      if (lds > 64 * 1024) return;
+      moe_plan_kernel<LP><<<dim3(1), dim3(1024), lds, s>>>(logits, row_stride, idx, weights, p, r);
+      done = true;
+    });
+  }
+  if (done) {
     NV_CHECK_LAUNCH();
     return NV_OK;
   }
   NV_CHECK_ARG(4 * scores <= 64 * 1024, "nv_moe_plan: the scores of %d outputs exceed the LDS", r.n);
-  moe_route_kernel<<<dim3((unsigned)((tokens + 3) / 4)), dim3(256), 4 * scores, s>>>(logits, row_stride, idx, weights, tokens, r);
+  launch_route(logits, row_stride, idx, weights, tokens, r, s);
   NV_CHECK_LAUNCH();
   moe_sort_kernel<<<dim3(1), dim3(1024), (size_t)experts * sizeof(int32_t), s>>>(p);
   NV_CHECK_LAUNCH();

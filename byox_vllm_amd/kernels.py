@@ -818,14 +818,14 @@ def moe_combine(y, slot_of, weights, shared=None, shared_gate=None, out=None):
 
 
 def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False, identity=0, correction=None, groups=0, keep_groups=0,
-             scale=1.0, self_weight=None):
+             scale=1.0, self_weight=None, row_weights=True):
     """Routing and ordering of fp32 router logits [T, >= experts].  With ``shared`` every token's last choice is expert
     number ``experts`` (weight 1): C = top + 1 choices and experts + 1 groups, else C = top.  The last ``identity`` of the
     experts + identity router outputs return their input: a choice of one owns no row (its sorted row is -1), and a token's
     weights of them are summed in ``self_weight`` fp32 [T].  ``correction`` fp32 [experts + identity] is added to the scores
     where they are compared; ``groups`` > 0: only the ``keep_groups`` best of that many groups of neighbours are chosen from;
     ``scale`` multiplies the weights.
-    -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C], sorted row of every
+    -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C] (None without ``row_weights``), sorted row of every
     choice int32 [T, C], the routed choices' weights fp32 [T, top])."""
     require_gpu(logits, "moe_plan")
     assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.size(1) >= experts + identity
@@ -839,7 +839,7 @@ def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False, identity=0, 
     weights = torch.empty(T, top, dtype=torch.float32, device=dev)
     offsets = torch.empty(experts + int(shared) + 1, dtype=torch.int32, device=dev)
     sorted_token = torch.empty(T * C, dtype=torch.int32, device=dev)
-    sorted_weight = torch.empty(T * C, dtype=torch.float32, device=dev)
+    sorted_weight = torch.empty(T * C, dtype=torch.float32, device=dev) if row_weights else None
     slot_of = torch.empty(T, C, dtype=torch.int32, device=dev)
     check(lib().nv_moe_plan(ptr(logits), logits.stride(0), T, experts, top, mode, int(shared), identity, ptr(correction), groups,
                             keep_groups, scale, ptr(idx), ptr(weights), ptr(offsets), ptr(sorted_token), ptr(sorted_weight),

@@ -116,7 +116,7 @@ class GroupedMixtureOfExperts(MixtureOfExperts):
         self_weight = torch.empty(T, dtype=torch.float32, device=h.device) if self.identity else None
         offsets, tokens, _, slot_of, weights = kernels.moe_plan(
             logits, E, top, self.route, identity=self.identity, correction=self.correction.data, groups=self.groups,
-            keep_groups=self.keep_groups, scale=self.scale, self_weight=self_weight)
+            keep_groups=self.keep_groups, scale=self.scale, self_weight=self_weight, row_weights=False)
         y = self.expert_rows(h, offsets, tokens)
         result = {"y": y, "slot_of": slot_of, "weights": weights}
         if self.identity:
