@@ -89,6 +89,9 @@ _PROTOS = {
     "nv_matrix_memory_state_size": (_i64, [_i, _i, _i]),
     "nv_matrix_memory": (_i, [_p, _i64, _i, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _p, _i64, _i, _i, _i, _i, _i, _i, _f, _f,
                               _p, _i, _f, _i, _i, _p]),
+    "nv_retention_step_ok": (_i, [_p, _i64, _i, _i, _i, _i, _p, _p, _i64, _i, _i]),
+    "nv_retention_step": (_i, [_p, _i64, _i, _i, _i, _i, _p, _p, _p, _p, _p, _p, _i, _f, _f, _f, _i, _p, _i64, _i, _i, _i, _i, _i,
+                               _p]),
     "nv_residual_pair": (_i, [_p, _p, _i64, _p, _p, _i64, _i, _i, _p]),
     "nv_latent_kv_store": (_i, [_p, _i64, _p, _p, _p, _f, _p, _p, _i64, _i, _i, _i, _i, _f, _i, _p]),
     "nv_latent_q_rope": (_i, [_p, _i64, _p, _p, _f, _p, _i64, _i, _i, _i, _i, _i, _i, _i, _p]),

@@ -294,6 +294,91 @@ __global__ __launch_bounds__(256) void matrix_memory_generic_kernel(MemArgs p) {
     for (int c = 0; c < copies; ++c) n_g[c * (p.dim + 1) + p.dim] = m_run;
 }
 
+// One token per request in the first form, with what follows it per head: o = S^T q after the update, divided by its root
+// mean square, times silu (or sigmoid) of the gate.  A workgroup owns one (head, request): lanes take four state columns
+// each, the key rows are dealt to the row groups of CG = vdim / 4 lanes, eight rows of state per thread in flight; the row
+// groups' partial o meet in LDS.
+constexpr int RS_THREADS = 512, RS_ROWS = 8;
+
+struct StepArgs {
+  MemArgs m;
+  int g_off, gate_silu;
+  float eps;
+  void* out;             // [tokens, out_rs] in the storage type
+  int64_t out_rs;
+};
+
+template <typename T>
+__global__ __launch_bounds__(RS_THREADS) void retention_step_kernel(StepArgs a) {
+  const MemArgs& p = a.m;
+  typedef typename Pack4<T>::type P;
+  extern __shared__ float4 lds4[];
+  __shared__ float red[32];
+  const int d = p.dim, vd = p.vdim, CG = vd >> 2, RG = RS_THREADS / CG;
+  float* so = reinterpret_cast<float*>(lds4);     // [RG][vd]
+  float* sq = so + RG * vd;                       // [d]
+  float* sk = sq + d;                             // [d]
+  const int h = blockIdx.x, b = blockIdx.y, tid = threadIdx.x;
+  const int t = p.cu_q[b];
+  if (p.cu_q[b + 1] <= t) return;
+  const int rg = tid / CG, c = (tid - rg * CG) * 4;
+  const bool on = rg < RG;
+  const bool fresh = p.past[b] == 0;
+  float* S_g = p.state + ((int64_t)p.slots[b] * p.H + h) * p.per_head;
+  const float* row = p.proj + (int64_t)t * p.proj_rs;
+  f32x4 s[RS_ROWS];
+  auto load = [&](int first) {
+#pragma unroll
+    for (int i = 0; i < RS_ROWS; ++i) {
+      const int r = first + i * RG;
+      s[i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+      if (on && !fresh && r < d) s[i] = *reinterpret_cast<const f32x4*>(S_g + (int64_t)r * vd + c);
+    }
+  };
+  load(rg);
+  const f32x4 v = on ? *reinterpret_cast<const f32x4*>(row + p.v_off + h * vd + c) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  const f32x4 z = on && rg == 0 ? *reinterpret_cast<const f32x4*>(row + a.g_off + h * vd + c) : f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  const float decay = p.decay[h];
+  const float* rot_row = p.rot + (int64_t)t * p.rot_dims;
+  for (int i = tid; i < d; i += RS_THREADS) {
+    sk[i] = turned(p, row + p.k_off + h * d, i, rot_row) * p.k_scale;
+    sq[i] = turned(p, row + p.q_off + h * d, i, rot_row) * p.q_scale;
+  }
+  __syncthreads();
+  f32x4 o = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  for (int first = rg; on && first < d; first += RS_ROWS * RG) {
+    if (first != rg) load(first);
+#pragma unroll
+    for (int i = 0; i < RS_ROWS; ++i) {
+      const int r = first + i * RG;
+      if (r >= d) continue;
+      const float k = sk[r], q = sq[r];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        s[i][e] = decay * s[i][e] + k * v[e];
+        o[e] += s[i][e] * q;
+      }
+      *reinterpret_cast<f32x4*>(S_g + (int64_t)r * vd + c) = s[i];
+    }
+  }
+  if (on) *reinterpret_cast<f32x4*>(so + rg * vd + c) = o;
+  __syncthreads();
+  float ss = 0.0f;
+  if (rg == 0) {
+    for (int g = 1; g < RG; ++g) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(so + g * vd + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[e] += x[e];
+    }
+    ss = o[0] * o[0] + o[1] * o[1] + o[2] * o[2] + o[3] * o[3];
+  }
+  const float inv = 1.0f / sqrtf(block_sum(ss, red) / (float)vd + a.eps);
+  if (rg != 0) return;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) o[e] *= inv * (a.gate_silu ? silu_f32(z[e]) : sigmoid_f32(z[e]));
+  *reinterpret_cast<P*>(reinterpret_cast<T*>(a.out) + (int64_t)t * a.out_rs + h * vd + c) = Pack4<T>::narrow(o);
+}
+
 // A workgroup of eight wavefronts owns one (head, request, slice of 64 state columns) and walks the request's tokens of this
 // step in chunks of C.  In LDS: the chunk's q and k rows (rotated, scaled), its values and the state TRANSPOSED (column
 // major: the products read four consecutive k numbers of a row or column per access), the decayed scores.  The state itself
@@ -646,6 +731,37 @@ extern "C" int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int 
       (size_t)(MM_TC * 2 * dmax + 3 * MM_TC + MM_TC * (threads / 64) + (cs > 1 ? cs * MM_TC * vdp : 0)) * sizeof(float);
   NV_CHECK_ARG(lds <= 64 * 1024 && threads <= 256, "nv_matrix_memory: launch plan out of range");
   NV_DISPATCH_T(dtype, launch_mem<T>(p, mode, dmax, cs, dim3(heads, num_seqs, slices), threads, lds, (hipStream_t)stream));
+  NV_CHECK_LAUNCH();
+  return NV_OK;
+}
+
+extern "C" int nv_retention_step_ok(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int g_off,
+                                    const float* state, const void* out, int64_t out_row_stride, int dim, int vdim) {
+  auto al16 = [](const void* q) { return (uintptr_t)q % 16 == 0; };
+  const size_t rg = RS_THREADS / (vdim >= 4 ? vdim / 4 : 1);
+  return vdim % 4 == 0 && vdim <= 1024 && (rg * vdim + 2 * (size_t)dim) * sizeof(float) <= 60 * 1024 && v_off % 4 == 0 &&
+         g_off % 4 == 0 && proj_row_stride % 4 == 0 && out_row_stride % 4 == 0 && al16(proj) && al16(state) && al16(out);
+}
+
+extern "C" int nv_retention_step(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int g_off,
+                                 const float* decay, float* state, const int32_t* cu_q, const int32_t* past_lens,
+                                 const int32_t* state_slots, const float* rot, int rot_dims, float q_scale, float k_scale,
+                                 float eps, int gate_silu, void* out, int64_t out_row_stride, int num_seqs, int heads, int dim,
+                                 int vdim, int dtype, nv_stream_t stream) {
+  NV_CHECK_ARG(proj && decay && state && cu_q && past_lens && state_slots && out, "nv_retention_step: null pointer");
+  NV_CHECK_ARG(dtype == NV_BF16 || dtype == NV_F32, "nv_retention_step: bad dtype %d", dtype);
+  NV_CHECK_ARG(heads > 0 && heads <= 65535 && dim > 0 && vdim > 0 && num_seqs >= 0 && num_seqs <= 65535 &&
+                   nv_retention_step_ok(proj, proj_row_stride, q_off, k_off, v_off, g_off, state, out, out_row_stride, dim, vdim),
+               "nv_retention_step: heads=%d dim=%d vdim=%d seqs=%d or an alignment this launch does not serve", heads, dim, vdim,
+               num_seqs);
+  NV_CHECK_ARG(rot_dims >= 0 && rot_dims % 2 == 0 && rot_dims <= dim && (rot_dims == 0 || rot),
+               "nv_retention_step: a rotation over %d of %d numbers needs its cosines and sines", rot_dims, dim);
+  if (num_seqs == 0) return NV_OK;
+  StepArgs a{{proj, proj_row_stride, q_off, k_off, v_off, 0, 0, nullptr, decay, state, cu_q, past_lens, state_slots, nullptr, 0,
+              heads, dim, vdim, dim * vdim, 0, q_scale, k_scale, 0.0f, rot, rot_dims},
+             g_off, gate_silu, eps, out, out_row_stride};
+  const size_t lds = ((size_t)(RS_THREADS / (vdim / 4)) * vdim + 2 * (size_t)dim) * sizeof(float);
+  NV_DISPATCH_T(dtype, retention_step_kernel<T><<<dim3(heads, num_seqs), dim3(RS_THREADS), lds, (hipStream_t)stream>>>(a));
   NV_CHECK_LAUNCH();
   return NV_OK;
 }

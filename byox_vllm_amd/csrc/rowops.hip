@@ -438,32 +438,44 @@ __device__ __forceinline__ uint32_t mix32(uint64_t x) {
   return (uint32_t)x;
 }
 
-__global__ __launch_bounds__(256) void sample_f32_kernel(const float* __restrict__ logits, int64_t rs,
+__global__ __launch_bounds__(1024) void sample_f32_kernel(const float* __restrict__ logits, int64_t rs,
                                                          const float* __restrict__ temperatures,
                                                          int64_t* __restrict__ tokens, int V, uint64_t seed) {
-  __shared__ float bv[256];
-  __shared__ int bi[256];
+  __shared__ float bv[1024];
+  __shared__ int bi[1024];
   const int row = blockIdx.x;
   const float temp = temperatures[row];
   const float* l = logits + row * rs;
   float best = -INFINITY;
   int arg = V;
-  for (int j = threadIdx.x; j < V; j += blockDim.x) {
-    float v = l[j];
-    if (temp > 0.0f) {
-      const uint32_t h = mix32(seed * 0x9E3779B97F4A7C15ULL + ((uint64_t)row << 32) + (uint64_t)j);
-      const float u = ((float)(h >> 8) + 0.5f) * (1.0f / 16777216.0f);
-      v = v / temp - logf(-logf(u));
+  constexpr int AHEAD = 8;             // logits of a thread that are on their way together
+  for (int base = threadIdx.x; base < V; base += AHEAD * blockDim.x) {
+    float x[AHEAD];
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) {
+      const int j = base + k * blockDim.x;
+      x[k] = j < V ? l[j] : 0.0f;
     }
-    if (v > best || arg == V) {
-      best = v;
-      arg = j;
+#pragma unroll
+    for (int k = 0; k < AHEAD; ++k) {
+      const int j = base + k * blockDim.x;
+      if (j >= V) break;
+      float v = x[k];
+      if (temp > 0.0f) {
+        const uint32_t h = mix32(seed * 0x9E3779B97F4A7C15ULL + ((uint64_t)row << 32) + (uint64_t)j);
+        const float u = ((float)(h >> 8) + 0.5f) * (1.0f / 16777216.0f);
+        v = v / temp - logf(-logf(u));
+      }
+      if (v > best || arg == V) {
+        best = v;
+        arg = j;
+      }
     }
   }
   bv[threadIdx.x] = best;
   bi[threadIdx.x] = arg;
   __syncthreads();
-  for (int o = 128; o > 0; o >>= 1) {
+  for (int o = 512; o > 0; o >>= 1) {
     if ((int)threadIdx.x < o) {
       const float v2 = bv[threadIdx.x + o];
       const int i2 = bi[threadIdx.x + o];
@@ -484,7 +496,7 @@ extern "C" int nv_sample_f32(const float* logits, int64_t row_stride, const floa
   NV_CHECK_ARG(logits && temperatures && tokens, "nv_sample_f32: null pointer");
   NV_CHECK_ARG(B >= 0 && V > 0, "nv_sample_f32: bad shape B=%d V=%d", B, V);
   if (B == 0) return NV_OK;
-  sample_f32_kernel<<<dim3((unsigned)B), dim3(256), 0, (hipStream_t)stream>>>(logits, row_stride, temperatures, tokens, V,
+  sample_f32_kernel<<<dim3((unsigned)B), dim3(1024), 0, (hipStream_t)stream>>>(logits, row_stride, temperatures, tokens, V,
                                                                               seed);
   NV_CHECK_LAUNCH();
   return NV_OK;

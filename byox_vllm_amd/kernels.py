@@ -677,6 +677,31 @@ def matrix_memory(proj, offsets, state, cu_q, past_lens, state_slots, heads, dim
     return out
 
 
+def retention_step(proj, offsets, decay, state, cu_q, past_lens, state_slots, heads, dim, vdim, *, eps, out_dtype, rot=None,
+                   q_scale=1.0, k_scale=1.0, gate_silu=False):
+    """matrix_memory (MEM_CONST) for steps of one token per request, then every head's result divided by its root mean
+    square and multiplied by the sigmoid (``gate_silu``: the SiLU) of its gate logits; ``offsets``: q | k | v | gate columns of
+    ``proj``.  -> rows [T, heads * vdim] in ``out_dtype``; None where the launch does not serve the sizes or alignments."""
+    require_gpu(proj, "retention_step")
+    T, B = proj.size(0), past_lens.numel()
+    assert proj.dtype == state.dtype == decay.dtype == torch.float32 and proj.stride(1) == 1 and state.is_contiguous()
+    assert state.shape[1:] == (heads, dim * vdim) and decay.numel() == heads and T == B
+    assert cu_q.dtype == past_lens.dtype == state_slots.dtype == torch.int32 and cu_q.numel() == B + 1 and state_slots.numel() == B
+    q_off, k_off, v_off, g_off = offsets
+    assert max(q_off + heads * dim, k_off + heads * dim, v_off + heads * vdim, g_off + heads * vdim) <= proj.size(1)
+    if rot is not None:
+        assert rot.dtype == torch.float32 and rot.is_contiguous() and rot.size(0) == T and rot.size(1) <= dim
+    out = torch.empty(T, heads * vdim, dtype=out_dtype, device=proj.device)
+    if not lib().nv_retention_step_ok(ptr(proj), proj.stride(0), q_off, k_off, v_off, g_off, ptr(state), ptr(out), out.stride(0),
+                                      dim, vdim):
+        return None
+    check(lib().nv_retention_step(ptr(proj), proj.stride(0), q_off, k_off, v_off, g_off, ptr(decay), ptr(state), ptr(cu_q),
+                                  ptr(past_lens), ptr(state_slots), ptr(rot), rot.size(1) if rot is not None else 0, q_scale,
+                                  k_scale, eps, int(gate_silu), ptr(out), out.stride(0), B, heads, dim, vdim, _code32(out_dtype),
+                                  stream()), "nv_retention_step")
+    return out
+
+
 def rotation_table(positions, inv_freq, out=None):
     """Cosines, then sines of position * inv_freq (float64 [half]) -> fp32 [T, 2 * half]; the angles are formed in double."""
     require_gpu(positions, "rotation_table")
@@ -825,8 +850,8 @@ def moe_plan(logits, experts, top, mode=ROUTE_CHOSEN, shared=False, identity=0, 
     weights of them are summed in ``self_weight`` fp32 [T].  ``correction`` fp32 [experts + identity] is added to the scores
     where they are compared; ``groups`` > 0: only the ``keep_groups`` best of that many groups of neighbours are chosen from;
     ``scale`` multiplies the weights.
-    -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C] (None without ``row_weights``), sorted row of every
-    choice int32 [T, C], the routed choices' weights fp32 [T, top])."""
+    -> (offsets int32 [groups + 1], token of every sorted row int32 [T * C], its weight fp32 [T * C] (None without
+    ``row_weights``), sorted row of every choice int32 [T, C], the routed choices' weights fp32 [T, top])."""
     require_gpu(logits, "moe_plan")
     assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.size(1) >= experts + identity
     assert correction is None or (correction.dtype == torch.float32 and correction.is_contiguous() and correction.is_cuda

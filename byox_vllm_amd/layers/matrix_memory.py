@@ -71,6 +71,10 @@ class _MatrixMemoryMixer(nn.Module):
     def _memory(self, proj, state, ctx, rot=None):
         raise NotImplementedError
 
+    def _step(self, proj, state, ctx, rot, dtype):
+        """One token per request: memory, norm and gate in one launch, where a mixer has one."""
+        return None
+
     norm_groups = 1
     gate_silu = False
 
@@ -87,6 +91,9 @@ class _MatrixMemoryMixer(nn.Module):
         ctx = get_context()
         if proj is None:
             proj = self.project(h)
+        y = self._step(proj, self.runs[run].state, ctx, rot, h.dtype) if ctx.max_seqlen_q == 1 else None
+        if y is not None:
+            return self.o(y, out_dtype=torch.float32)
         o = self._memory(proj, self.runs[run].state, ctx, rot)
         g = self.at["g"]
         y = kernels.group_rms_norm_f32(o, self.norm.data if self.norm is not None else None, self.norm_groups, self.eps,
@@ -125,6 +132,11 @@ class Retention(_MatrixMemoryMixer):
                                      ctx.past_lens, ctx.state_slots, self.heads, self.dim, self.vdim, self.mode,
                                      decay=self.decay, k_scale=self.dim ** -0.5, rot=rot,
                                      max_q=ctx.max_seqlen_q)
+
+    def _step(self, proj, state, ctx, rot, dtype):
+        return kernels.retention_step(proj, tuple(self.at[s] for s in "qkvg"), self.decay, state, ctx.cu_seqlens_q, ctx.past_lens,
+                                      ctx.state_slots, self.heads, self.dim, self.vdim, eps=self.eps, out_dtype=dtype, rot=rot,
+                                      k_scale=self.dim ** -0.5, gate_silu=True)
 
 
 class MLSTM(_MatrixMemoryMixer):

@@ -451,6 +451,16 @@ int nv_matrix_memory(const float* proj, int64_t proj_row_stride, int q_off, int 
                      const int32_t* state_slots, float* out, int64_t out_row_stride, int num_seqs, int heads, int dim,
                      int vdim, int mode, int silu, float q_scale, float k_scale, const float* rot, int rot_dims, float cap,
                      int max_q, int dtype, nv_stream_t stream);
+/* Steps of one token per request in mode 0 with what follows per head, in one launch: o divided by its root mean square,
+ * times sigmoid (gate_silu: SiLU) of the gate logits at columns g_off + h * vdim of proj, rows in the storage type.  Serves
+ * what nv_retention_step_ok admits (value sizes of a multiple of 4, 16-byte aligned arrays). */
+int nv_retention_step_ok(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int g_off,
+                         const float* state, const void* out, int64_t out_row_stride, int dim, int vdim);
+int nv_retention_step(const float* proj, int64_t proj_row_stride, int q_off, int k_off, int v_off, int g_off,
+                      const float* decay, float* state, const int32_t* cu_q, const int32_t* past_lens,
+                      const int32_t* state_slots, const float* rot, int rot_dims, float q_scale, float k_scale, float eps,
+                      int gate_silu, void* out, int64_t out_row_stride, int num_seqs, int heads, int dim, int vdim, int dtype,
+                      nv_stream_t stream);
 /* out[t] (2 * half fp32 numbers): cosines, then sines of positions[t] * inv_freq[i], formed in double. */
 int nv_rotation_table(const int64_t* positions, const double* inv_freq, float* out, int64_t tokens, int half,
                       nv_stream_t stream);

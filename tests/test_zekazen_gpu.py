@@ -274,6 +274,45 @@ def test_retention_batch_of_unequal_requests():
             assert float((O.retention(q, k * 0.25, v, torch.tensor(decay, dtype=F64)) - want)[-1, 0].abs().max()) > 1.0
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,d,dv,rot", [(2, 16, 24, 8), (1, 10, 4, 2), (3, 72, 80, 0), (2, 128, 128, 128), (1, 264, 300, 16), (2, 40, 1024, 40)])
+@pytest.mark.parametrize("silu", [False, True])
+def test_single_token_steps_with_norm_and_gate(dtype, H, d, dv, rot, silu):
+    """The one-launch form of decoded tokens: a fresh request and two that continue, token after token."""
+    from byox_vllm_amd import kernels
+    T, eps = 12, 1e-3
+    g = torch.Generator().manual_seed(d + dv)
+    decay = torch.tensor([0.05, 0.93, 1.0][:H])
+    offs = (1, 2 + H * d, 4 + 2 * H * d + (-2 * H * d) % 4, 8 + 2 * H * d + (-2 * H * d) % 4 + H * dv)
+    cols = offs[3] + H * dv + 4 - (offs[3] + H * dv) % 4
+    proj = {r: torch.randn(T, cols, generator=g) for r in range(3)}
+    freq = torch.tensor([100.0 ** (-2.0 * i / rot) for i in range(rot // 2)], dtype=F64, device=DEV) if rot else None
+    state = torch.full((4, H, d * dv), float("nan"), device=DEV)
+    start, got = [0, 5, 1], {r: [] for r in range(3)}
+    table = lambda p: kernels.rotation_table(p.to(DEV), freq) if rot else None     # noqa: E731
+    for r in (1, 2):                                       # what these two hold already
+        n = start[r]
+        kernels.matrix_memory(_dev(proj[r][:n]), offs[:3], state, _i32([0, n]), _i32([0]), _i32([r + 1]), H, d, dv, kernels.MEM_CONST,
+                              decay=_dev(decay), k_scale=0.3, rot=table(torch.arange(n)), max_q=n)
+    for i in range(T - 5):
+        pos = torch.tensor([s + i for s in start])
+        rows = torch.stack([proj[r][pos[r]] for r in range(3)])
+        y = kernels.retention_step(_dev(rows), offs, _dev(decay), state, _i32([0, 1, 2, 3]), pos.int().to(DEV), _i32([1, 2, 3]), H, d, dv,
+                                   eps=eps, out_dtype=dtype, rot=table(pos), k_scale=0.3, gate_silu=silu)
+        assert y is not None and y.dtype == dtype
+        for r in range(3):
+            got[r].append(y[r].float().cpu())
+    for r in range(3):
+        n = start[r] + T - 5
+        x = proj[r][:n].double()
+        q, k = (O.rotate(x[:, o:o + H * d].reshape(n, H, d), torch.arange(n), rot, 100.0) for o in offs[:2])
+        o = O.retention(q, k * 0.3, x[:, offs[2]:offs[2] + H * dv].reshape(n, H, dv), decay.double())
+        z = x[:, offs[3]:offs[3] + H * dv]
+        want = O.rms(o, eps).reshape(n, -1) * (O.silu(z) if silu else torch.sigmoid(z))
+        _close(torch.stack(got[r]), want[start[r]:], 1e-5 if dtype == torch.float32 else 8e-3)
+    assert torch.isnan(state[0]).all()
+
+
 def test_activated_keys_in_chunks_equal_steps(monkeypatch):
     """Lightning attention's memory (q, k and v through SiLU, no rotation) takes the chunks too."""
     H, d, dv = 2, 64, 72
