@@ -12,7 +12,7 @@
 // other, so slices need nothing from each other but each keeps its own copy of the normaliser and the maximum; launches
 // of many requests give a workgroup all slices of a head instead - and walks the request's tokens of this step in order, starting from the slot (or from zero when
 // the request has no tokens behind it) and leaving the state there: a prompt portion, the next portion and single
-// decoded tokens all go through this one kernel (states that do not fit a workgroup's registers: a slow general kernel
+// decoded tokens can all go through this one kernel (states that do not fit a workgroup's registers: a slow general kernel
 // that keeps the state in its slot).  The results are fp32 rows; the norm and gate that follow them span
 // heads or not, depending on the design, and run in nv_group_rmsnorm_f32.
 //
@@ -22,7 +22,8 @@
 // of the chunk are a scalar recurrence that one thread walks while the others stage.  Thread d < dim also carries n[d];
 // the sixteen n . q meet through wavefront sums.
 //
-// Prompts in the first form take retention_chunk_kernel instead: with ONE constant decay per head, C tokens at once are
+// Single tokens in the first form can take their head's norm and gate along in one launch (retention_step_kernel).
+// Prompts in the first form take retention_chunk_kernel where sizes and alignments allow: with ONE constant decay per head, C tokens at once are
 // matrix products on the fp32 matrix cores (v_mfma_f32_16x16x4_f32, true fp32),
 //   o_i = decay^(i+1) S^T q_i + sum_(j <= i) decay^(i-j) (q_i . k_j) v_j,
 //   S  <- decay^n S + sum_j decay^(n-1-j) k_j v_j^T,

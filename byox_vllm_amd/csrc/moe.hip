@@ -25,9 +25,9 @@ struct RouteArgs {
   const float* correction;   // [n] added to the scores where they are compared (not to the weights), or null
   int groups, keep;          // > 0: n / groups neighbours form a group; only the `keep` groups with the best member count
   float scale;               // factor on the weights
-  // the choice compares scores (kept in LDS, n numbers per wavefront) and not plain logits
+  // the choice compares scores and not plain logits
   __host__ __device__ bool scored() const { return correction != nullptr || groups > 0; }
-  // numbers of LDS per wavefront: scores, then best members of the groups, each padded to whole 16 bytes
+  // numbers of LDS per token at work: what is compared, then best members of the groups, each padded to whole 16 bytes
   __host__ __device__ int n4() const { return (n + 3) & ~3; }
   __host__ __device__ int lds_words() const { return n <= 128 || scored() ? n4() + ((groups + 3) & ~3) : 0; }
 };

@@ -91,12 +91,12 @@ def random_config(seed: int):
     rng = random.Random(seed)
     layers = []
     for _ in range(rng.randint(2, 6)):
-        d, dv = rng.choice([16, 20, 24, 32, 48, 64, 80, 96]), rng.choice([8, 12, 16, 24, 40, 64, 80])
+        d, dv = rng.choice([16, 20, 24, 32, 48, 64, 88, 104]), rng.choice([8, 12, 16, 24, 40, 64, 72])
         if rng.random() < 0.5:
             H = rng.choice([1, 2, 3, 5])
             rot = rng.choice([0, 2, d // 2, d]) // 2 * 2
             mixer = retention(H, d, dv, [rng.choice([0.3, 0.9, 1.0 - 2.0 ** -rng.randint(3, 12)]) for _ in range(H)],
-                              (rng.choice([100.0, 1e4, 1e6]), rot) if rot else None)
+                              (rng.choice([100.0, 1e4, 3e5]), rot) if rot else None)
         else:
             G = rng.choice([1, 2, 3, 4])
             mixer = attention(G * rng.choice([1, 2, 3, 4]), G, d, dv, rng.choice([d ** -0.5, 0.3, 1.0]), rng.choice([1, 2, 3, 4, 5]),
@@ -107,7 +107,7 @@ def random_config(seed: int):
             keep = rng.randint(1, count)
             identity = rng.randint(0, count * size - 1)
             mlp = moe(count * size - identity, rng.randint(1, min(4, keep * size)), rng.choice([16, 20, 40, 64]),
-                      (count, keep), identity, rng.choice([0.5, 1.0, 2.5]))
+                      (count, keep), identity, rng.choice([0.5, 1.0, 2.4]))
         layers.append((mixer, mlp))
     return config(rng.choice([97, 250, 300]), rng.choice([64, 72, 100, 144, 192]), layers, eps=rng.choice([1e-5, 1e-6, 1e-3]))
 
